@@ -14,7 +14,7 @@ from __future__ import annotations
 from collections.abc import Sequence
 from dataclasses import dataclass
 
-from turboserve_amd.parts.base import CacheNeed, FixedState, PagedKV
+from turboserve_amd.parts.base import CacheNeed, FixedState, PagedKV, SharedKV, shares_pages
 
 
 @dataclass(frozen=True)
@@ -40,18 +40,37 @@ class PageGroup:
 class CacheLayout:
     groups: tuple[PageGroup, ...]
     state_entries: tuple[tuple[int, FixedState], ...]
-    #: per schedule entry: ("pages", group, unit) | ("state", index) | ("reads", entry) | None, or,
-    #: for an entry whose mixer has several needs, a tuple of such units in the order of the needs
+    #: per schedule entry: ("pages", group, unit) | ("shared", group, unit) | ("state", index) | ("reads", entry) | None,
+    #: or, for an entry whose mixer has several needs, a tuple of such units in the order of the needs
     entry_units: tuple[tuple | None, ...]
 
     @classmethod
     def from_needs(cls, needs: Sequence[CacheNeed], reads: Sequence[int | None]) -> "CacheLayout":
         """``needs[i]``: what schedule entry ``i`` owns (one need, or a tuple of needs);
-        ``reads[i]``: the earlier entry whose cache it reads instead."""
+        ``reads[i]``: the earlier entry whose cache it reads instead, or whose pages a ``SharedKV`` among
+        its needs means."""
         keys: list[tuple] = []
         members: list[list[int]] = []
         states: list[tuple[int, FixedState]] = []
         units: list[tuple | None] = []
+
+        def shared_pages(entry: int, need: SharedKV) -> tuple[int, int]:
+            """The group and member of the pages that the entry named by ``reads`` owns, if they are what the reader takes them for."""
+            source = reads[entry]
+            if source is None:
+                raise ValueError(f"schedule entry {entry} asks for another entry's pages and names none")
+            owned = units[source] if units[source] is not None and units[source] and not isinstance(units[source][0], str) else (units[source],)
+            pages = [unit for unit in owned if unit is not None and unit[0] == "pages"]
+            if len(pages) != 1:
+                raise ValueError(f"schedule entry {entry} asks for the pages of entry {source}, which owns {len(pages)} sets of them")
+            _, group, member = pages[0]
+            heads, dim, window, value_width, chunk, _ = keys[group]
+            if (heads, dim, value_width) != (need.num_kv_heads, need.head_dim, need.value_width):
+                raise ValueError(f"schedule entry {entry} reads {need.num_kv_heads} heads of {need.head_dim}/{need.value_width} where entry "
+                                 f"{source} keeps {heads} of {dim}/{value_width}")
+            if chunk is not None or (window is not None and (need.window is None or need.window > window)):
+                raise ValueError(f"schedule entry {entry} reads keys that entry {source} does not keep")
+            return group, member
 
         def unit_of(entry: int, need) -> tuple | None:
             if isinstance(need, PagedKV):
@@ -65,12 +84,14 @@ class CacheLayout:
             if isinstance(need, FixedState):
                 states.append((entry, need))
                 return ("state", len(states) - 1)
+            if isinstance(need, SharedKV):
+                return ("shared", *shared_pages(entry, need))
             if need is None:
                 return None
             raise TypeError(f"schedule entry {entry} declares an unknown cache need {need!r}")
 
         for entry, need in enumerate(needs):
-            if reads[entry] is not None:
+            if reads[entry] is not None and not shares_pages(need):
                 units.append(("reads", reads[entry]))
             elif isinstance(need, (tuple, list)):
                 units.append(tuple(unit_of(entry, one) for one in need))
@@ -81,7 +102,9 @@ class CacheLayout:
 
     @classmethod
     def from_model(cls, model) -> "CacheLayout":
-        return cls.from_needs(model.cache_needs(), [call.cache_of for call in model.plan.schedule])
+        needs = model.cache_needs()
+        reads: list[int | None] = [call.cache_of for call in model.plan.schedule]
+        return cls.from_needs(needs, reads + [None] * (len(needs) - len(reads)))  # (an embedding with state has an entry behind the calls)
 
     def windows(self) -> list[int | None]:
         return [group.window for group in self.groups]

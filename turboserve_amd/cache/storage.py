@@ -74,8 +74,9 @@ class CacheStorage:
     def _unit_view(self, unit: tuple | None, writable: bool) -> CacheView:
         if unit is None:
             return None
-        if unit[0] == "pages":
-            _, group, member = unit
+        if unit[0] in ("pages", "shared"):
+            kind, group, member = unit
+            writable = writable and kind == "pages"
             spec = self.layout.groups[group]
             pages = self.num_pages[group]
             return PagedKVView(

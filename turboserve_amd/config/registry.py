@@ -74,3 +74,8 @@ def _ensure_builtin() -> None:
         from turboserve_amd.models.legavik import legavik_plan
 
         register_architecture("Legavik", LegavikConfig.from_dict, legavik_plan)
+    if "Lukelix" not in ARCHITECTURES:
+        from turboserve_amd.config.lukelix_config import LukelixConfig
+        from turboserve_amd.models.lukelix import lukelix_plan
+
+        register_architecture("Lukelix", LukelixConfig.from_dict, lukelix_plan)

@@ -17,7 +17,8 @@
 // rest pass), `values_are_keys` (there are no value columns: the values are the key heads as projected,
 // before norm and rotation), `temp_coef`/`temp_every` (a query at position p is multiplied by 1 + temp_coef
 // ln(floor((p + 1) / temp_every) + 1), last of all), `tail` (a row of the projection holds that many columns
-// more behind the heads, which are left alone).
+// more behind the heads, which are left alone), `neighbours` (the pairs turned together are (2i, 2i + 1) instead of (i, i +
+// rot_dims/2)).  kv_heads may be 0: the projection holds queries only, and nothing is stored.
 //
 // Values may be blended with another layer's values of the same tokens before they are stored
 // (ValueBlend): `keep` [T, Hkv Dv] 32-bit, if given, receives this layer's values as projected;
@@ -37,6 +38,7 @@ struct HeadShape {
   float temp_coef;
   int temp_every;
   int tail;  // columns of a projection's row behind the heads, read by others
+  int neighbours;
 };
 
 struct ValueBlend {
@@ -138,10 +140,11 @@ head_norm_store_kernel(T* q_out, long q_stride, const P* proj, int splits, size_
     for (int c = 0; c < PER_LANE; ++c) {
       const int d = lane + c * TS_WAVE;
       if (d < turned) {
-        const int i = d < half ? d : d - half;
-        const float x1 = held[wave][i], x2 = held[wave][i + half];
+        const bool first = shape.neighbours ? (d & 1) == 0 : d < half;
+        const int i = shape.neighbours ? d >> 1 : first ? d : d - half;  // the pair's angle
+        const float x1 = held[wave][shape.neighbours ? d & ~1 : i], x2 = held[wave][shape.neighbours ? d | 1 : i + half];
         const float cv = cos_table[at + i], sv = sin_table[at + i];
-        x[c] = d < half ? __builtin_fmaf(x1, cv, -(x2 * sv)) : __builtin_fmaf(x2, cv, x1 * sv);
+        x[c] = first ? __builtin_fmaf(x1, cv, -(x2 * sv)) : __builtin_fmaf(x2, cv, x1 * sv);
       }
     }
   }
@@ -168,16 +171,17 @@ head_norm_store_kernel(T* q_out, long q_stride, const P* proj, int splits, size_
   }
 }
 
-// The same for many tokens (prompt portions): bfloat16 in and out, no partial sums, no rotation,
-// head size a multiple of 8 and at most 128.  Sixteen lanes per (token, q or k head), eight
+// The same for many tokens (prompt portions): bfloat16 in and out, no partial sums, no rotation or one of
+// neighbouring pairs (a multiple of 8 elements of a head), head size a multiple of 8 and at most 128.  Sixteen lanes per (token, q or k head), eight
 // elements a lane with one 16-byte load and one 16-byte store; the sum of squares is formed over
 // the sixteen lanes of a row by data-parallel moves.  Per element the arithmetic of the kernel
 // above.
 __global__ void __launch_bounds__(256)
 head_norm_store_rows_kernel(bf16_t* q_out, long q_stride, const bf16_t* proj, bf16_t* __restrict__ k_pages,
                             const bf16_t* __restrict__ q_gain, const bf16_t* __restrict__ k_gain, float eps,
-                            float gain_offset, const int* __restrict__ slots, int tokens, int heads, int kv_heads,
-                            int dim, int vdim, int block_size) {
+                            float gain_offset, const float* __restrict__ cos_table, const float* __restrict__ sin_table,
+                            const int* __restrict__ positions, int turned, const int* __restrict__ slots, int tokens, int heads,
+                            int kv_heads, int dim, int vdim, int block_size) {
   const int qk_heads = heads + kv_heads;
   const long items = (long)tokens * qk_heads;
   const long asked = (long)blockIdx.x * 16 + threadIdx.x / 16;
@@ -213,6 +217,17 @@ head_norm_store_rows_kernel(bf16_t* q_out, long q_stride, const bf16_t* proj, bf
     const float r = rsqrtf(ss / (float)dim + eps);
 #pragma unroll
     for (int e = 0; e < 8; ++e) x[e] = x[e] * r * (gain_offset + g[e]);
+  }
+  if (cos_table && piece * 8 < turned) {  // the lane's four pairs
+    const size_t at = (size_t)positions[t] * (turned / 2) + piece * 4;
+    const float4 cv = *reinterpret_cast<const float4*>(cos_table + at), sv = *reinterpret_cast<const float4*>(sin_table + at);
+    const float cs[4] = {cv.x, cv.y, cv.z, cv.w}, sn[4] = {sv.x, sv.y, sv.z, sv.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float x1 = x[2 * e], x2 = x[2 * e + 1];
+      x[2 * e] = __builtin_fmaf(x1, cs[e], -(x2 * sn[e]));
+      x[2 * e + 1] = __builtin_fmaf(x2, cs[e], x1 * sn[e]);
+    }
   }
   bf16_t* dst = nullptr;
   if (h < heads) {
@@ -282,11 +297,13 @@ static void launch_head_norm_store(void* q_out, long q_stride, const void* proj,
   const bool aligned = ((uintptr_t)q_out | (uintptr_t)proj | (uintptr_t)k_pages | (uintptr_t)q_gain | (uintptr_t)k_gain) % 16 == 0 &&
                        q_stride % 8 == 0 && vdim % 8 == 0;
   const bool plain = (!shape.normed || q_gain) && !shape.norm_after && !shape.values_are_keys && shape.temp_coef == 0.f && shape.tail == 0;
-  if (std::is_same<T, bf16_t>::value && std::is_same<P, bf16_t>::value && splits == 1 && !cos_table && dim % 8 == 0 &&
+  const int turned = shape.rot_dims > 0 ? shape.rot_dims : dim;
+  const bool in_lanes = !cos_table || (shape.neighbours && turned % 8 == 0 && ((uintptr_t)cos_table | (uintptr_t)sin_table) % 16 == 0);
+  if (std::is_same<T, bf16_t>::value && std::is_same<P, bf16_t>::value && splits == 1 && in_lanes && dim % 8 == 0 &&
       dim <= 128 && !few && aligned && plain)
     hipLaunchKernelGGL(head_norm_store_rows_kernel, dim3((unsigned)((items + 15) / 16)), dim3(256), 0, stream, (bf16_t*)q_out,
                        q_stride, (const bf16_t*)proj, (bf16_t*)k_pages, (const bf16_t*)q_gain, (const bf16_t*)k_gain, eps,
-                       gain_offset, slots, tokens, heads, kv_heads, dim, vdim, block_size);
+                       gain_offset, cos_table, sin_table, positions, turned, slots, tokens, heads, kv_heads, dim, vdim, block_size);
   else
     hipLaunchKernelGGL((head_norm_store_kernel<T, P>), dim3((unsigned)((items + HNS_WAVES - 1) / HNS_WAVES)),
                        dim3(64 * HNS_WAVES), 0, stream, (T*)q_out, q_stride, (const P*)proj, splits, (size_t)split_stride,
@@ -304,18 +321,19 @@ extern "C" int ts_head_norm_store(void* q_out, long q_stride, const void* proj, 
                                   const float* sin_table, const int* positions, const int* slots, int tokens,
                                   int heads, int kv_heads, int dim, int vdim, int block_size, int dtype,
                                   float* v_keep, const float* v_other, float v_weight, int normed, int norm_after,
-                                  int rot_dims, int values_are_keys, float temp_coef, int temp_every, int tail, hipStream_t stream) {
+                                  int rot_dims, int values_are_keys, float temp_coef, int temp_every, int tail, int neighbours,
+                                  hipStream_t stream) {
   if (tokens == 0) return TS_OK;
-  const HeadShape shape = {normed, norm_after, rot_dims, values_are_keys, temp_coef, temp_every, tail};
+  const HeadShape shape = {normed, norm_after, rot_dims, values_are_keys, temp_coef, temp_every, tail, neighbours};
   if (rot_dims < 0 || rot_dims > dim || (rot_dims & 1) || (values_are_keys && vdim != dim) || (temp_coef != 0.f && temp_every < 1) || tail < 0)
     return TS_ERR_ARG;
   if ((v_keep || v_other) && !slots) return TS_ERR_ARG;  // values are only walked where they are stored
   const ValueBlend blend = {v_keep, v_other, v_weight};
-  if (!q_out || !proj || !positions || heads < 1 || kv_heads < 1 || dim < 1 || dim > HNS_MAX_DIM || vdim < 1 ||
+  if (!q_out || !proj || !positions || heads < 1 || kv_heads < 0 || (kv_heads == 0 && slots) || dim < 1 || dim > HNS_MAX_DIM || vdim < 1 ||
       block_size < 1 || splits < 1 || kv_heads > 65535)
     return TS_ERR_ARG;
   if ((cos_table == nullptr) != (sin_table == nullptr) || (cos_table && rot_dims == 0 && (dim & 1))) return TS_ERR_ARG;
-  if ((q_gain == nullptr) != (k_gain == nullptr)) return TS_ERR_ARG;
+  if (kv_heads > 0 && (q_gain == nullptr) != (k_gain == nullptr)) return TS_ERR_ARG;
   if (slots && (!k_pages || !v_pages)) return TS_ERR_ARG;
   if (dtype == TS_F32)
     launch_head_norm_store<float, float>(q_out, q_stride, proj, splits, split_stride, k_pages, v_pages, q_gain, k_gain, eps, gain_offset, cos_table, sin_table, positions, slots, tokens, heads, kv_heads, dim, vdim, block_size, blend, shape, stream);

@@ -5,8 +5,8 @@
 // elements apart that are added up here; the convolved channels are its columns first_col .. first_col +
 // channels - 1.  y_t[c] = sum_j taps[c][j] * u_(t - K + 1 + j)[c], where u is the request's own sequence of
 // inputs: those of this step's earlier rows, and before them the K - 1 inputs the request's state slot
-// holds (state [slots, K - 1, channels] 32-bit, oldest first; zero for a request that starts).  With
-// `activation` 1 the result goes through silu.  The result is [T, channels] of type T, or 32-bit.
+// holds (state [slots, K - 1, channels] 32-bit, oldest first; zero for a request that starts).  A `bias` [channels],
+// where given, is added; with `activation` 1 the result then goes through silu.  The result is [T, channels] of type T, or 32-bit.
 //
 // ts_short_conv computes every row of the step and leaves the state alone; ts_short_conv_carry, launched
 // behind it, moves each request's last K - 1 inputs into its slot.  In a step whose requests all bring one
@@ -35,7 +35,7 @@ __device__ __forceinline__ float sc_input(const P* p, int splits, size_t stride)
 template <typename T, typename P, typename O>
 __global__ void __launch_bounds__(256)
 short_conv_kernel(O* __restrict__ out, const P* __restrict__ proj, int splits, size_t split_stride, int width, int first_col,
-                  int channels, const T* __restrict__ taps, int k,
+                  int channels, const T* __restrict__ taps, const T* __restrict__ bias, int k,
                   float* state, const int* __restrict__ state_slots, const int* __restrict__ token_seq,
                   const int* __restrict__ query_start_loc, int activation, int single) {
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
@@ -60,6 +60,7 @@ short_conv_kernel(O* __restrict__ out, const P* __restrict__ proj, int splits, s
     y = fmaf(to_float(taps[(size_t)c * k + j]), u, y);
   }
   if (single && k > 1) held[(size_t)(k - 2) * channels] = mine;
+  if (bias) y += to_float(bias[c]);
   if (activation == 1) y = y / (1.f + expf(-y));
   out[(size_t)t * channels + c] = from_float<O>(y);
 }
@@ -70,7 +71,7 @@ short_conv_kernel(O* __restrict__ out, const P* __restrict__ proj, int splits, s
 template <typename O, int K>
 __global__ void __launch_bounds__(256)
 short_conv_rows_kernel(O* __restrict__ out, const bf16_t* __restrict__ proj, int width, int first_col, int channels,
-                       const bf16_t* __restrict__ taps, const float* __restrict__ state,
+                       const bf16_t* __restrict__ taps, const bf16_t* __restrict__ bias, const float* __restrict__ state,
                        const int* __restrict__ state_slots, const int* __restrict__ token_seq,
                        const int* __restrict__ query_start_loc, int activation) {
   const int c = 4 * (blockIdx.y * blockDim.x + threadIdx.x);
@@ -109,6 +110,10 @@ short_conv_rows_kernel(O* __restrict__ out, const bf16_t* __restrict__ proj, int
 #pragma unroll
     for (int e = 0; e < 4; ++e) y[e] = fmaf(w[e * K + j], u[e], y[e]);
   }
+  if (bias) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) y[e] += to_float(bias[c + e]);
+  }
 #pragma unroll
   for (int e = 0; e < 4; ++e)
     if (activation == 1) y[e] = y[e] / (1.f + expf(-y[e]));
@@ -145,7 +150,7 @@ short_conv_carry_kernel(float* __restrict__ state, const P* __restrict__ proj, i
 
 // dtype: the run's type (taps, and the projection unless it is partial sums); out_f32: a 32-bit result.
 extern "C" int ts_short_conv(void* out, int out_f32, const void* proj, int in_f32, int splits, long split_stride, int width,
-                             int first_col, int channels, const void* taps, int k, float* state,
+                             int first_col, int channels, const void* taps, const void* bias, int k, float* state,
                              const int* state_slots, const int* token_seq, const int* query_start_loc, int tokens,
                              int activation, int single, int dtype, hipStream_t stream) {
   if (tokens == 0) return TS_OK;
@@ -161,10 +166,10 @@ extern "C" int ts_short_conv(void* out, int out_f32, const void* proj, int in_f3
   case K:                                                                                                                \
     if (out_f32)                                                                                                         \
       hipLaunchKernelGGL((short_conv_rows_kernel<float, K>), wide, block, 0, stream, (float*)out, (const bf16_t*)proj, width,       \
-                         first_col, channels, (const bf16_t*)taps, state, state_slots, token_seq, query_start_loc, activation);  \
+                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation);  \
     else                                                                                                                 \
       hipLaunchKernelGGL((short_conv_rows_kernel<bf16_t, K>), wide, block, 0, stream, (bf16_t*)out, (const bf16_t*)proj, width,     \
-                         first_col, channels, (const bf16_t*)taps, state, state_slots, token_seq, query_start_loc, activation);  \
+                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation);  \
     break;
     switch (k) {
       SC_ROWS(1) SC_ROWS(2) SC_ROWS(3) SC_ROWS(4) SC_ROWS(5) SC_ROWS(6) SC_ROWS(7) SC_ROWS(8)
@@ -174,7 +179,7 @@ extern "C" int ts_short_conv(void* out, int out_f32, const void* proj, int in_f3
   }
 #define SC_GO(T, P, O)                                                                                                   \
   hipLaunchKernelGGL((short_conv_kernel<T, P, O>), grid, block, 0, stream, (O*)out, (const P*)proj, splits, (size_t)split_stride, \
-                     width, first_col, channels, (const T*)taps, k, state, state_slots, token_seq, query_start_loc, activation, single)
+                     width, first_col, channels, (const T*)taps, (const T*)bias, k, state, state_slots, token_seq, query_start_loc, activation, single)
   if (dtype == TS_F32) SC_GO(float, float, float);
   else if (dtype == TS_BF16 && in_f32 && out_f32) SC_GO(bf16_t, float, float);
   else if (dtype == TS_BF16 && in_f32) SC_GO(bf16_t, float, bf16_t);

@@ -37,8 +37,11 @@ MODULES: dict[str, tuple[str, ...]] = {
         "mixer_store.hip",
         "linear_state.hip",
         "delta_state.hip",
+        "selective_state.hip",
         "short_conv.hip",
         "tanh_norm.hip",
+        "layer_norm.hip",
+        "bigram.hip",
         "moe.hip",
         "attention_generic.hip",
         "attention_tiles.hip",

@@ -80,7 +80,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "ts_head_norm_store": [c_void_p, c_long, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_int, c_float, c_int,
-                               c_int, c_void_p],
+                               c_int, c_int, c_void_p],
         "ts_span_norm_store": [c_void_p, c_long, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_float, c_float, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
         "ts_latent_store": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float, c_void_p,
@@ -93,10 +93,21 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "ts_add_tanh_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float, c_void_p, c_int,
                              c_int, c_int, c_void_p, c_int, c_long, c_void_p],
         "ts_tanh_cap": [c_void_p, c_long, c_float, c_void_p],
-        "ts_short_conv": [c_void_p, c_int, c_void_p, c_int, c_int, c_long, c_int, c_int, c_int, c_void_p, c_int, c_void_p,
+        "ts_short_conv": [c_void_p, c_int, c_void_p, c_int, c_int, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "ts_short_conv_carry": [c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                                 c_int, c_int, c_void_p],
+        "ts_selective_walk": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_void_p,
+                              c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_selective_pieces": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_void_p,
+                                c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_selective_carry": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_gated_group_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_float, c_int, c_int, c_int,
+                                c_int, c_void_p],
+        "ts_add_layer_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float, c_float, c_void_p,
+                              c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+        "ts_embed_bigram": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                            c_int, c_int, c_int, c_int, c_void_p],
         "ts_delta_prepare": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int,
                              c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
         "ts_delta_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
@@ -672,6 +683,7 @@ class Ops:
         values_are_keys: bool = False,
         query_temperature: tuple[float, int] | None = None,
         tail: int = 0,
+        neighbours: bool = False,
     ) -> tuple[torch.Tensor, int]:
         """Per-head norm of the q and k heads of the fused projection ``[T, Hq D + Hkv D + Hkv Dv]``
         (``x * rsqrt(mean(x^2) + eps) * (gain_offset + gain)`` in 32-bit, the gain ``[D]`` shared by
@@ -686,7 +698,9 @@ class Ops:
         ``[capacity, R/2]`` with ``R < D`` turn the first ``R`` elements of a head only; ``values_are_keys``:
         the projection is ``[T, Hq D + Hkv D]`` and the values are the key heads as projected;
         ``query_temperature = (coef, every)``: a query at position ``p`` is multiplied by ``1 + coef ln(floor((p
-        + 1) / every) + 1)``; ``tail``: a row of the projection holds that many columns more behind the heads."""
+        + 1) / every) + 1)``; ``tail``: a row of the projection holds that many columns more behind the heads;
+        ``neighbours``: the pairs turned together are ``(2i, 2i + 1)`` instead of ``(i, i + R/2)``.  With ``kv_heads =
+        0`` the projection holds queries only (and ``k_gain`` is not looked at)."""
         _gpu(proj, k_pages, v_pages, q_gain, k_gain, positions, slots, cos, sin, keep_values)
         _i32(positions, "positions")
         _i32(slots, "slots")
@@ -698,7 +712,8 @@ class Ops:
             _need(dtype is not None, "partial sums need the run dtype")
         is_f32, splits, stride = self._partials(proj, tokens, width, run_dtype, "projection")
         _need(1 <= head_dim <= ATTENTION_MAX_HEAD_DIM and value_dim >= 1, "head sizes outside what the kernel takes")
-        _need((q_gain is None) == (k_gain is None), "both gains or none")
+        _need(kv_heads >= 1 or slots is None, "without key heads nothing is stored")
+        _need(kv_heads == 0 or (q_gain is None) == (k_gain is None), "both gains or none")
         for gain in (q_gain, k_gain):
             if gain is not None:
                 _need(gain.shape == (head_dim,) and gain.dtype == run_dtype and gain.is_contiguous(),
@@ -732,7 +747,8 @@ class Ops:
             _ptr(k_gain), float(eps), float(gain_offset), _ptr(cos), _ptr(sin), _ptr(positions), _ptr(slots), tokens,
             heads, kv_heads, head_dim, value_dim, block_size, dtype_code(run_dtype), _ptr(keep_values), _ptr(other),
             float(weight), 1 if normed else 0, 1 if norm_after else 0, 0 if cos is None else 2 * cos.shape[1],
-            1 if values_are_keys else 0, float(coef), int(every), int(tail), self.stream()), "ts_head_norm_store")
+            1 if values_are_keys else 0, float(coef), int(every), int(tail), 1 if neighbours else 0, self.stream()),
+            "ts_head_norm_store")
         return q_out, q_stride
 
     # -- stores and stream steps of other mixers ------------------------------------------------
@@ -1004,14 +1020,14 @@ class Ops:
 
     def short_conv(self, proj: torch.Tensor, first_col: int, taps: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor,
                    token_seq: torch.Tensor, query_start_loc: torch.Tensor, *, tokens: int, num_seqs: int, dtype: torch.dtype,
-                   silu: bool = False, out_float32: bool = False) -> torch.Tensor:
+                   silu: bool = False, out_float32: bool = False, bias: torch.Tensor | None = None) -> torch.Tensor:
         """A short causal convolution over time on the ``C`` columns of ``proj`` from ``first_col`` on (``taps [C,
         K]``: ``y_t = sum_j taps[:, j] u_(t - K + 1 + j)``), continuing every request from the ``K - 1`` inputs its
         state slot holds (``state [slots, max(K - 1, 1), C]`` 32-bit, oldest first) and leaving its last ``K - 1``
         inputs there (by a second launch; in a step whose requests all bring one token the first launch does it).
         ``proj`` is ``[T, W]`` of the run dtype or 32-bit partial sums.  Returns ``[T, C]`` of the run dtype (32-bit
-        with ``out_float32``), through ``silu`` if asked."""
-        _gpu(proj, taps, state, state_slots, token_seq, query_start_loc)
+        with ``out_float32``), plus ``bias [C]`` where given, through ``silu`` if asked."""
+        _gpu(proj, taps, bias, state, state_slots, token_seq, query_start_loc)
         _i32(state_slots, "state_slots")
         _i32(token_seq, "token_seq")
         _i32(query_start_loc, "query_start_loc")
@@ -1020,6 +1036,8 @@ class Ops:
         channels, k = taps.shape
         _need(taps.dtype == dtype and taps.is_contiguous() and 1 <= k <= 8 and 0 <= first_col and first_col + channels <= width,
               "taps must be [C, K] of the run dtype, K up to 8, over columns of the projection")
+        _need(bias is None or (bias.shape == (channels,) and bias.dtype == dtype and bias.is_contiguous()),
+              "the convolution's bias must be [C] of the run dtype")
         _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 3
               and state.shape[1:] == (max(k - 1, 1), channels), "the state must be float32 [slots, K - 1, C]")
         _need(token_seq.numel() >= tokens and query_start_loc.numel() >= num_seqs + 1 and state_slots.numel() >= num_seqs,
@@ -1031,7 +1049,7 @@ class Ops:
         # Every request brings one token: the launch that convolves also moves the state on.
         single = tokens == num_seqs
         _check(self.core.ts_short_conv(_ptr(out), 1 if wide else 0, _ptr(proj), is_f32, splits, stride, width, first_col, channels,
-                                       _ptr(taps), k, _ptr(state), _ptr(state_slots), _ptr(token_seq), _ptr(query_start_loc),
+                                       _ptr(taps), _ptr(bias), k, _ptr(state), _ptr(state_slots), _ptr(token_seq), _ptr(query_start_loc),
                                        tokens, 1 if silu else 0, 1 if single else 0, code, self.stream()), "ts_short_conv")
         if single:
             return out
@@ -1094,6 +1112,133 @@ class Ops:
                                          _ptr(gain), float(eps), tokens, heads, value_dim, code, float(scale), out_stride,
                                          self.stream()), "ts_delta_finish")
         return y
+
+    # -- layer norm, two-table embedding ---------------------------------------------------------
+
+    def add_layer_norm(self, residual: torch.Tensor, pending: torch.Tensor | None, dtype: torch.dtype, rows: torch.Tensor | None = None, *,
+                       norm: tuple[torch.Tensor, torch.Tensor, float] | None = None,
+                       pending_norm: tuple[torch.Tensor, torch.Tensor, float, float] | None = None) -> torch.Tensor:
+        """``residual += p`` in 32-bit (in place) and the sum in ``dtype``, rounded once: through a layer norm where
+        ``norm = (weight [H], bias [H], eps)`` is given, as it is otherwise.  ``p`` is ``pending`` (``[T, H]`` of
+        ``dtype`` or ``[S, T, H]`` 32-bit partial sums), with ``pending_norm = (weight, bias, eps, scale)`` first
+        normalised on its own and multiplied by ``scale``, in 32-bit.  With ``rows`` only those rows, and ``residual`` is left
+        alone."""
+        _gpu(residual, pending, rows)
+        _i32(rows, "rows")
+        _need(residual.dim() == 2 and residual.dtype == torch.float32 and residual.is_contiguous(),
+              "residual must be contiguous float32 [T, H]")
+        tokens, hidden = residual.shape
+        _need(hidden <= 16384, "layer norms take rows of up to 16,384 elements")
+        is_f32, splits, stride = (0, 1, 0)
+        if pending is not None:
+            is_f32, splits, stride = self._partials(pending, tokens, hidden, dtype, "pending")
+        _need(pending_norm is None or pending is not None, "a norm on the pending output needs one")
+        for rule in (norm, pending_norm):
+            for t in () if rule is None else rule[:2]:
+                _gpu(t)
+                _need(t.shape == (hidden,) and t.dtype == dtype and t.is_contiguous(), "a layer norm's weight and bias must be [H] of the run dtype")
+        w, b, eps = (None, None, 0.0) if norm is None else norm
+        post_w, post_b, post_eps, post_scale = (None, None, 0.0, 1.0) if pending_norm is None else pending_norm
+        out_rows = tokens if rows is None else rows.numel()
+        y = self.rows_buffer(out_rows, hidden, dtype, residual.device)
+        _check(self.core.ts_add_layer_norm(_ptr(y), _ptr(residual), _ptr(pending), is_f32, splits, stride, _ptr(post_w), _ptr(post_b),
+                                           float(post_eps), float(post_scale), _ptr(w), _ptr(b), float(eps), _ptr(rows), out_rows, hidden,
+                                           dtype_code(dtype), self.stream()), "ts_add_layer_norm")
+        return y
+
+    def embed_bigram(self, table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, held: torch.Tensor, state_slots: torch.Tensor,
+                     token_seq: torch.Tensor, query_start_loc: torch.Tensor, *, num_seqs: int, mul_prev: int, mul_cur: int) -> torch.Tensor:
+        """``float32 [T, H]``: row ``ids[t]`` of ``table [V, H]`` plus row ``(prev * mul_prev + ids[t] * mul_cur) mod B`` of
+        ``pairs [B + 1, H]``, ``prev`` the token before it in its request; a request's first token takes row ``B``.  The
+        token before a step's first is what the request's slot of ``held [slots, 1]`` (int32: an id plus one, 0 for none)
+        holds, and the request's last token is left there."""
+        _gpu(table, pairs, ids, held, state_slots, token_seq, query_start_loc)
+        for t, what in ((ids, "ids"), (held, "held"), (state_slots, "state_slots"), (token_seq, "token_seq"), (query_start_loc, "query_start_loc")):
+            _i32(t, what)
+        tokens, (vocab, hidden), buckets = ids.numel(), table.shape, pairs.shape[0] - 1
+        _need(table.is_contiguous() and pairs.is_contiguous() and pairs.dim() == 2 and pairs.shape[1] == hidden and buckets >= 1
+              and pairs.dtype == table.dtype, "the tables must be contiguous [V, H] and [B + 1, H] of one dtype")
+        _need(held.dim() == 2 and held.shape[1] == 1 and token_seq.numel() >= tokens and query_start_loc.numel() >= num_seqs + 1
+              and state_slots.numel() >= num_seqs, "row ranges and slots of every request")
+        out = torch.empty((tokens, hidden), dtype=torch.float32, device=table.device)
+        _check(self.core.ts_embed_bigram(_ptr(out), _ptr(table), _ptr(pairs), _ptr(ids), _ptr(held), _ptr(state_slots), _ptr(token_seq),
+                                         _ptr(query_start_loc), tokens, num_seqs, hidden, vocab, buckets, int(mul_prev) % buckets,
+                                         int(mul_cur) % buckets, dtype_code(table.dtype), self.stream()), "ts_embed_bigram")
+        return out
+
+    # -- a selective state space -----------------------------------------------------------------
+
+    #: Tokens of a piece when long portions are cut up to run side by side (the kernels' own constant).
+    selective_piece = 128
+    #: Portions of up to this many tokens are walked, longer ones (bfloat16 runs) cut into pieces.
+    selective_walk_tokens = 32
+
+    @staticmethod
+    def selective_pieces_supported(dtype: torch.dtype, state_dim: int, value_dim: int) -> bool:
+        """Whether long portions can be cut into pieces on the matrix cores: bfloat16, state rows of up to 256,
+        state rows and columns both multiples of 8 (16-byte accesses)."""
+        return dtype == torch.bfloat16 and state_dim <= 256 and state_dim % 8 == 0 and value_dim % 8 == 0
+
+    def selective_state(self, u: torch.Tensor, proj: torch.Tensor, dt_at: int, dt_bias: torch.Tensor, a_log: torch.Tensor,
+                        skip: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, query_start_loc: torch.Tensor, *,
+                        num_seqs: int, heads: int, groups: int, state_dim: int, value_dim: int, dtype: torch.dtype,
+                        plan: tuple | None = None) -> torch.Tensor:
+        """A selective state space over a step: per head and request a 32-bit state ``S [N, P]`` (``state [slots, H, P,
+        N]``) that every token decays and adds to: ``dt = softplus(d + dt_bias)``, ``S <- exp(-exp(a_log) dt) S + dt B
+        x^T``, ``y = S^T C + skip x``.  ``u [T, H P + 2 G N]`` of ``dtype`` holds the step's convolved ``x | B | C`` (head
+        ``h`` uses group ``h // (H / G)``), ``d`` is the ``H`` columns of ``proj`` from ``dt_at`` on.  Returns ``y [T, H P]``
+        32-bit.  Without a ``plan`` every request is walked; ``plan = (pieces, carries, n_pieces, n_requests)`` (int32
+        device tensors from :meth:`linear_state_pieces`, for the requests from 0 on) cuts the first ``n_requests`` into
+        pieces of :attr:`selective_piece` tokens that run side by side, and the requests behind them are walked."""
+        _gpu(u, proj, dt_bias, a_log, skip, state, state_slots, query_start_loc)
+        _i32(state_slots, "state_slots")
+        _i32(query_start_loc, "query_start_loc")
+        tokens, width = proj.shape[-2], proj.shape[-1]
+        is_f32, splits, stride = self._partials(proj, tokens, width, dtype, "projection")
+        _need(u.dtype == dtype and u.is_contiguous() and u.shape == (tokens, heads * value_dim + 2 * groups * state_dim),
+              "the convolved x | B | C must be [T, H P + 2 G N] of the run dtype")
+        _need(heads % groups == 0 and 1 <= state_dim <= 512 and 0 <= dt_at and dt_at + heads <= width, "sizes the selective state does not take")
+        for t in (dt_bias, a_log, skip):
+            _need(t.shape == (heads,) and t.dtype == torch.float32 and t.is_contiguous(), "dt_bias, a_log and skip must be float32 [H]")
+        _need(state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (heads, value_dim, state_dim),
+              "the state must be float32 [slots, H, P, N]")
+        _need(query_start_loc.numel() >= num_seqs + 1 and state_slots.numel() >= num_seqs, "row ranges and slots of every request")
+        y = torch.empty((tokens, heads * value_dim), dtype=torch.float32, device=u.device)
+        steps = (_ptr(proj), is_f32, splits, stride, width, dt_at, _ptr(dt_bias), _ptr(a_log), _ptr(skip))
+        first = 0
+        if plan is not None:
+            pieces, carries, n_pieces, first = plan
+            _i32(pieces, "pieces")
+            _i32(carries, "carries")
+            _need(self.selective_pieces_supported(dtype, state_dim, value_dim) and first <= num_seqs, "a geometry that is not cut into pieces")
+            piece_state = torch.empty((n_pieces, heads, value_dim, state_dim), dtype=torch.float32, device=u.device)
+            piece_decay = torch.empty((n_pieces, heads), dtype=torch.float32, device=u.device)
+            for mode in (0, 1):
+                _check(self.core.ts_selective_pieces(_ptr(y), _ptr(piece_state), _ptr(piece_decay), _ptr(u), *steps, _ptr(pieces), n_pieces,
+                                                     heads, groups, state_dim, value_dim, mode, self.stream()), "ts_selective_pieces")
+                if mode == 0:
+                    _check(self.core.ts_selective_carry(_ptr(state), _ptr(state_slots), _ptr(carries), _ptr(piece_state), _ptr(piece_decay),
+                                                        first, heads, state_dim, value_dim, self.stream()), "ts_selective_carry")
+        _check(self.core.ts_selective_walk(_ptr(y), _ptr(state), _ptr(u), 1 if dtype == torch.float32 else 0, *steps, _ptr(state_slots),
+                                           _ptr(query_start_loc), first, num_seqs - first, heads, groups, state_dim, value_dim,
+                                           dtype_code(dtype), self.stream()), "ts_selective_walk")
+        return y
+
+    def gated_group_norm(self, y: torch.Tensor, proj: torch.Tensor, z_at: int, gain: torch.Tensor, eps: float, parts: int,
+                         dtype: torch.dtype) -> torch.Tensor:
+        """``[T, W]`` of ``dtype``: the 32-bit ``y [T, W]`` times ``silu`` of the ``W`` columns of ``proj`` from ``z_at`` on, every one
+        of ``parts`` equal parts of a row divided by its own root mean square (``eps`` inside the root), times ``gain [W]``."""
+        _gpu(y, proj, gain)
+        tokens, width = y.shape
+        is_f32, splits, stride = self._partials(proj, tokens, proj.shape[-1], dtype, "projection")
+        _need(y.dtype == torch.float32 and y.is_contiguous() and gain.shape == (width,) and gain.dtype == dtype and gain.is_contiguous(),
+              "y must be float32 [T, W] and the gain [W] of the run dtype")
+        _need(1 <= parts and width % parts == 0 and 0 <= z_at and z_at + width <= proj.shape[-1], "equal parts, and the gate's columns inside the projection")
+        _need(width // parts <= 16384, "parts of up to 16,384 elements")
+        out = self.rows_buffer(tokens, width, dtype, y.device)
+        _check(self.core.ts_gated_group_norm(_ptr(out), _ptr(y), _ptr(proj), is_f32, splits, stride, proj.shape[-1], z_at, _ptr(gain), float(eps),
+                                             tokens, parts, width // parts, dtype_code(dtype), self.stream()), "ts_gated_group_norm")
+        return out
 
     # -- routed feed-forward --------------------------------------------------------------------
 

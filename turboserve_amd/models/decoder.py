@@ -27,6 +27,7 @@ from turboserve_amd.parts.base import (
     Runtime,
     StreamStep,
     TensorSpec,
+    shares_pages,
 )
 from turboserve_amd.parts.registry import build_part
 
@@ -42,7 +43,8 @@ class LayerSpec:
 @dataclass(frozen=True)
 class LayerCall:
     """One entry of the run order: which layer runs and, optionally, the index of an EARLIER
-    entry whose cache it reads (it then writes nothing).  ``enter``: a stream step (kind,
+    entry whose cache it reads (it then writes nothing there; a mixer that asks for ``SharedKV`` reads that
+    entry's pages and keeps what state it asks for itself).  ``enter``: a stream step (kind,
     parameters and the checkpoint prefix of its tensors) that acts on the residual stream right
     before this call: what a model adds when a pass through repeated layers begins."""
 
@@ -175,21 +177,29 @@ class DecoderModel:
         return merge_step_fields(asked)
 
     def cache_needs(self) -> list[CacheNeed]:
-        """What each schedule entry needs a cache for (``None``: nothing, or it reads another's)."""
+        """What each schedule entry needs a cache for (``None``: nothing, or it reads another's) and, behind
+        them, what the embedding needs one for, if it does."""
         needs: list[CacheNeed] = []
         for call in self.plan.schedule:
             need = self.blocks[call.layer].mixer.cache_need()
-            needs.append(None if call.cache_of is not None else need)
+            needs.append(None if call.cache_of is not None and not shares_pages(need) else need)
+        if self.embedding.cache_need() is not None:
+            needs.append(self.embedding.cache_need())
         return needs
 
     # -- the pass -----------------------------------------------------------------------------
 
     def forward(self, token_ids: torch.Tensor, ctx, caches: Sequence[CacheView]) -> ResidualStream:
         """Embedding and every scheduled layer call over the step's flat tokens
-        (model.py:105-107).  ``caches[i]`` is the view of schedule entry ``i``."""
-        if len(caches) != len(self.plan.schedule):
-            raise ValueError(f"{len(caches)} cache views for {len(self.plan.schedule)} scheduled layer calls")
-        stream = ResidualStream(self.embedding.forward(token_ids, ctx))
+        (model.py:105-107).  ``caches[i]`` is the view of schedule entry ``i``; an embedding that carries
+        state has its view behind them."""
+        calls = len(self.plan.schedule)
+        carried = self.embedding.cache_need() is not None
+        if len(caches) != calls + (1 if carried else 0):
+            raise ValueError(f"{len(caches)} cache views for {calls} scheduled layer calls"
+                             f"{' and an embedding with state' if carried else ''}")
+        start = self.embedding.forward(token_ids, ctx, caches[calls]) if carried else self.embedding.forward(token_ids, ctx)
+        stream = ResidualStream(start)
         # The embedding's output is kept apart only where a stream step adds it in again later.
         origin = self.runtime.ops.copy_float32(stream.residual) if self.keeps_origin else None
         for call, cache, enter in zip(self.plan.schedule, caches, self.enter_steps):

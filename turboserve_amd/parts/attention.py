@@ -8,7 +8,7 @@ from collections.abc import Mapping
 import torch
 
 from turboserve_amd.kernels.ops import attention_geometry_error
-from turboserve_amd.parts.base import CacheNeed, FixedState, Mixer, PagedKV, PagedKVView, PartSpec, Runtime, TensorSpec
+from turboserve_amd.parts.base import CacheNeed, FixedState, Mixer, PagedKV, PagedKVView, PartSpec, Runtime, SharedKV, TensorSpec
 from turboserve_amd.parts.registry import build_part, register_mixer
 
 
@@ -65,7 +65,9 @@ class GroupedQueryAttention(Mixer):
     K]`` under ``<tensor name>.<s>``, the last column the current token's); the request's last ``K - 1``
     projected rows are state that the cache keeps beside the pages.  ``query_temperature = {"coef": c,
     "every": n}``: the query at position ``p`` is multiplied by ``1 + c ln(floor((p + 1) / n) + 1)`` behind
-    norm and encoding.  ``names``: the tensor
+    norm and encoding.  ``own_keys=False``: there are no key and value tensors (matrices, biases, convolutions,
+    norms); the layer's queries read the keys and values of the layer call that its schedule entry names
+    (``LayerCall.cache_of``), as that call's pages hold them.  ``names``: the tensor
     names under the part's prefix of ``q, k, v, o`` (biases: the same with ``weight`` replaced by
     ``bias``) and of the two gains."""
 
@@ -97,6 +99,7 @@ class GroupedQueryAttention(Mixer):
         gate_name: str | None = None,
         conv: Mapping | None = None,
         query_temperature: Mapping | None = None,
+        own_keys: bool = True,
     ) -> None:
         super().__init__(prefix, runtime)
         # Refused here, when the model is put together, not at the first step after the weights
@@ -117,6 +120,9 @@ class GroupedQueryAttention(Mixer):
         self.values_are_keys = bool(values_are_keys)
         if self.values_are_keys and (self.value_dim != self.head_dim or value_mix is not None):
             raise ValueError(f"{prefix or 'attention'}: values that are the keys have the keys' size and are not mixed")
+        self.own_keys = bool(own_keys)
+        if not self.own_keys and (self.values_are_keys or value_mix is not None or span_norm is not None or keep_first or chunk is not None):
+            raise ValueError(f"{prefix or 'attention'}: a layer without keys of its own has no say in how keys and values are made or kept")
         self.keep_first = int(keep_first)
         if self.keep_first < 0 or (self.keep_first > 0 and (window is None or chunk is not None)):
             raise ValueError(f"{prefix or 'attention'}: kept first keys go with a window and without chunks")
@@ -160,8 +166,10 @@ class GroupedQueryAttention(Mixer):
         self.names = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
                       "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", **(names or {})}
         self.q_size = self.num_heads * self.head_dim
-        self.kv_size = self.num_kv_heads * self.head_dim
-        self.v_size = 0 if self.values_are_keys else self.num_kv_heads * self.value_dim
+        #: Key heads in the projection (none where another layer's keys are read).
+        self.projected_kv_heads = self.num_kv_heads if self.own_keys else 0
+        self.kv_size = self.projected_kv_heads * self.head_dim
+        self.v_size = 0 if self.values_are_keys else self.projected_kv_heads * self.value_dim
         self.out_size = self.num_heads * self.value_dim
         self.conv_weight: torch.Tensor | None = None
         self.q_gain: torch.Tensor | None = None
@@ -172,14 +180,19 @@ class GroupedQueryAttention(Mixer):
         self.o_bias_tensor: torch.Tensor | None = None
 
     def cache_need(self) -> CacheNeed:
-        pages = PagedKV(self.num_kv_heads, self.head_dim, self.window,
-                        None if self.value_dim == self.head_dim else self.value_dim, self.chunk, self.keep_first)
+        value_dim = None if self.value_dim == self.head_dim else self.value_dim
+        if self.own_keys:
+            pages = PagedKV(self.num_kv_heads, self.head_dim, self.window, value_dim, self.chunk, self.keep_first)
+        else:
+            pages = SharedKV(self.num_kv_heads, self.head_dim, value_dim, self.window)
         if self.conv_taps is None:
             return pages
         # The request's last projected rows, 32-bit, beside its pages.
         return (pages, FixedState((max(self.conv_taps - 1, 1), self.q_size + self.kv_size + self.v_size), torch.float32))
 
     def _projections(self) -> tuple[str, ...]:
+        if not self.own_keys:
+            return ("q",)
         return ("q", "k") if self.values_are_keys else ("q", "k", "v")
 
     def is_capturable(self) -> bool:
@@ -211,7 +224,8 @@ class GroupedQueryAttention(Mixer):
         if self.head_norm_eps is not None and self.head_norm_gain:
             init = "zeros" if self.head_norm_offset == 1.0 else "ones"
             specs[self.name(self.names["q_norm"])] = TensorSpec((self.head_dim,), init=init)
-            specs[self.name(self.names["k_norm"])] = TensorSpec((self.head_dim,), init=init)
+            if self.own_keys:
+                specs[self.name(self.names["k_norm"])] = TensorSpec((self.head_dim,), init=init)
         if self.span_norm_eps is not None:
             init = "zeros" if self.span_norm_offset == 1.0 else "ones"
             specs[self.name(self.names["q_norm"])] = TensorSpec((self.q_size,), init=init)
@@ -248,7 +262,7 @@ class GroupedQueryAttention(Mixer):
             self.o_bias_tensor = tensors[self.name(self._bias("o"))].contiguous()
         if (self.head_norm_eps is not None and self.head_norm_gain) or self.span_norm_eps is not None:
             self.q_gain = tensors[self.name(self.names["q_norm"])].contiguous()
-            self.k_gain = tensors[self.name(self.names["k_norm"])].contiguous()
+            self.k_gain = None if not self.own_keys else tensors[self.name(self.names["k_norm"])].contiguous()
         if self.sink_name is not None:
             self.sink_scores = tensors[self.name(self.sink_name)].float().contiguous()
         if self.value_mix is not None and not self.value_mix.get("source"):
@@ -307,7 +321,7 @@ class GroupedQueryAttention(Mixer):
             else:
                 more["values"] = {"blend": (ctx.carried[key], self.mix_weight)}
         q, q_stride = self.position.encode_and_store(
-            qkv, self.num_heads, self.num_kv_heads, self.head_dim, ctx, cache, **more
+            qkv, self.num_heads, self.projected_kv_heads, self.head_dim, ctx, cache, **more
         )
         attended = self.attend(q, q_stride, ctx, cache)
         if self.gate_name is not None:

@@ -81,9 +81,31 @@ class FixedState:
     dtype: torch.dtype = torch.float32
 
 
-#: What a mixer asks of the cache: nothing, pages, fixed-size state, or several of these (a
+@dataclass(frozen=True)
+class SharedKV:
+    """A mixer's need for keys and values that another layer call owns: the one its schedule entry
+    names (``LayerCall.cache_of``).  It gets that call's pages, read-only, and may ask for state of its
+    own beside them.  The sizes must be what those pages hold, and the owner must keep every key the reader
+    sees (``window`` keys; ``None``: all of them)."""
+
+    num_kv_heads: int
+    head_dim: int
+    value_dim: int | None = None
+    window: int | None = None
+
+    @property
+    def value_width(self) -> int:
+        return self.head_dim if self.value_dim is None else self.value_dim
+
+
+#: What a mixer asks of the cache: nothing, pages, another call's pages, fixed-size state, or several of these (a
 #: layer that keeps pages and a state of its own gets one view for each, in the order asked).
-CacheNeed = PagedKV | FixedState | None | tuple
+CacheNeed = PagedKV | SharedKV | FixedState | None | tuple
+
+
+def shares_pages(need: "CacheNeed") -> bool:
+    """Whether a need names another call's pages (alone or among others)."""
+    return any(isinstance(one, SharedKV) for one in (need if isinstance(need, tuple) else (need,)))
 
 
 @dataclass
@@ -139,8 +161,19 @@ class ResidualStream:
     also: torch.Tensor | None = None
     #: ``(gain [H], eps, scale)``: ``pending`` is normalised on its own before it is added, so what the
     #: stream gets is ``scale * gain * pending / rms(pending)``, in 32-bit (a block with a norm behind
-    #: each part); the norm that adds ``pending`` does this in the same pass.
-    pending_norm: tuple | None = None
+    #: each part); or a :class:`PendingLayerNorm`.  The norm that adds ``pending`` does this in the same pass.
+    pending_norm: "tuple | PendingLayerNorm | None" = None
+
+
+@dataclass(frozen=True)
+class PendingLayerNorm:
+    """The rule of a pending output that passes a layer norm before it is added: the stream gets ``scale *
+    ((p - mean) / sqrt(variance + eps) * weight + bias)``, in 32-bit."""
+
+    weight: torch.Tensor
+    bias: torch.Tensor
+    eps: float
+    scale: float
 
 
 # ---------------------------------------------------------------------------------------------
@@ -213,9 +246,9 @@ class Norm(Part):
         stream is left as it is."""
         raise NotImplementedError
 
-    def pending_rule(self, scale: float) -> tuple:
+    def pending_rule(self, scale: float) -> "tuple | PendingLayerNorm":
         """This norm as the rule of a pending output (``ResidualStream.pending_norm``): ``(gain, eps,
-        scale)``, for a block that normalises a part's output before the residual sum."""
+        scale)`` or a :class:`PendingLayerNorm`, for a block that normalises a part's output before the residual sum."""
         raise NotImplementedError(f"{type(self).__name__} cannot be applied to a pending output")
 
 
@@ -244,7 +277,8 @@ class PositionEncoding(Part):
         ``head_norm = (q_gain [D], k_gain [D], eps, gain_offset)`` (every q and k head is divided
         by its root mean square and multiplied by ``gain_offset + gain`` before the encoding), ``shape``
         (a mapping of what else the per-head store takes: ``normed`` without gains, ``norm_after`` the
-        encoding, ``values_are_keys``, ``query_temperature``, ``tail`` columns behind the heads)."""
+        encoding, ``values_are_keys``, ``query_temperature``, ``tail`` columns behind the heads).  A projection of queries
+        only has ``num_kv_heads = 0``: nothing is stored."""
         raise NotImplementedError
 
     def score_slopes(self, num_heads: int) -> torch.Tensor | None:
@@ -263,6 +297,11 @@ class PositionEncoding(Part):
 
 class Embedding(Part):
     """Token ids -> what the first layer's residual stream starts as."""
+
+    def cache_need(self) -> CacheNeed:
+        """As a mixer's: what an embedding that looks at earlier tokens of a request carries from step to
+        step.  ``forward`` then gets the view as a third argument."""
+        return None
 
     def forward(self, token_ids: torch.Tensor, ctx: "StepContext") -> torch.Tensor:
         """``token_ids [T]`` int32 -> 32-bit ``[T, H]``."""

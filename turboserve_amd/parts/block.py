@@ -147,7 +147,8 @@ class SandwichBlock(Block):
     with the norm's rule beside it (``stream.pending_norm``), and the next norm that carries the
     residual sum (this block's, the next block's or the head's) normalises it, scales it and adds it,
     all in 32-bit, before it normalises the sum.  A block without a feed-forward
-    (``feed_forward=None``) is its first half alone.  The four norms' checkpoint names under the
+    (``feed_forward=None``) is its first half alone.  ``pre_norm``: another norm in front of the parts than
+    behind them (``plain_sum``: none, ``h += norm_a2(mixer(h)); h += norm_b2(feed_forward(h))``).  The four norms' checkpoint names under the
     block's prefix are ``mixer_norm_name``, ``mixer_post_name``, ``ff_norm_name``, ``ff_post_name``."""
 
     def __init__(
@@ -158,6 +159,7 @@ class SandwichBlock(Block):
         mixer: PartSpec,
         feed_forward: PartSpec | None,
         norm: PartSpec,
+        pre_norm: PartSpec | None = None,
         residual_scale: float = 1.0,
         mixer_name: str = "mix",
         ff_name: str = "mlp",
@@ -168,12 +170,13 @@ class SandwichBlock(Block):
     ) -> None:
         super().__init__(prefix, runtime)
         self.residual_scale = float(residual_scale)
-        self.mixer_norm = build_part("norm", norm, self.name(mixer_norm_name), runtime)
+        pre_norm = norm if pre_norm is None else pre_norm
+        self.mixer_norm = build_part("norm", pre_norm, self.name(mixer_norm_name), runtime)
         self.mixer = build_part("mixer", mixer, self.name(mixer_name), runtime)
         self.mixer_post = build_part("norm", norm, self.name(mixer_post_name), runtime)
         self.ff_norm = self.feed_forward = self.ff_post = None
         if feed_forward is not None:
-            self.ff_norm = build_part("norm", norm, self.name(ff_norm_name), runtime)
+            self.ff_norm = build_part("norm", pre_norm, self.name(ff_norm_name), runtime)
             self.feed_forward = build_part("feed_forward", feed_forward, self.name(ff_name), runtime)
             self.ff_post = build_part("norm", norm, self.name(ff_post_name), runtime)
 

@@ -8,7 +8,7 @@ from collections.abc import Mapping
 
 import torch
 
-from turboserve_amd.parts.base import Embedding, Head, PartSpec, ResidualStream, Runtime, TensorSpec
+from turboserve_amd.parts.base import CacheNeed, Embedding, FixedState, FixedStateView, Head, PartSpec, ResidualStream, Runtime, TensorSpec
 from turboserve_amd.parts.registry import build_part, register_embedding, register_head
 
 
@@ -75,6 +75,37 @@ class SinusoidTokenTable(TokenTable):
     def forward(self, token_ids: torch.Tensor, ctx) -> torch.Tensor:
         self.ensure_capacity(ctx.max_context_len)
         return self.runtime.ops.embed_positions(self.weight, token_ids, ctx.positions, self.at)
+
+
+@register_embedding("token_table_bigram")
+class BigramTokenTable(TokenTable):
+    """A token's row of the table plus a row of a second table ``[buckets + 1, H]`` (``pairs_name``, a full
+    checkpoint name) hashed from the token and the one before it in its request, ``(previous * mul_prev + token *
+    mul_cur) mod buckets``; a request's first token takes the last row.  Summed in 32-bit.  The request's last token is
+    state: its id plus one in the request's slot, 0 where the request starts."""
+
+    def __init__(self, prefix: str, runtime: Runtime, *, vocab_size: int, hidden_size: int, buckets: int, mul_prev: int, mul_cur: int,
+                 pairs_name: str, weight_name: str = "weight") -> None:
+        super().__init__(prefix, runtime, vocab_size=vocab_size, hidden_size=hidden_size, weight_name=weight_name)
+        self.buckets, self.mul_prev, self.mul_cur = int(buckets), int(mul_prev), int(mul_cur)
+        if not 1 <= self.buckets < 2**31 - 1:
+            raise ValueError(f"{prefix}: {self.buckets} buckets")
+        self.pairs_name = pairs_name
+        self.pairs: torch.Tensor | None = None
+
+    def cache_need(self) -> CacheNeed:
+        return FixedState((1,), torch.int32)
+
+    def tensor_specs(self) -> dict[str, TensorSpec]:
+        return {**super().tensor_specs(), self.pairs_name: TensorSpec((self.buckets + 1, self.hidden_size))}
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        super().load(tensors)
+        self.pairs = tensors[self.pairs_name].contiguous()
+
+    def forward(self, token_ids: torch.Tensor, ctx, cache: FixedStateView) -> torch.Tensor:
+        return self.runtime.ops.embed_bigram(self.weight, self.pairs, token_ids, cache.state, ctx.state_slots, ctx.token_seq,
+                                             ctx.query_start_loc, num_seqs=ctx.num_seqs, mul_prev=self.mul_prev, mul_cur=self.mul_cur)
 
 
 @register_head("norm_linear")

@@ -48,6 +48,22 @@ def interpolated_frequencies(head_dim: int, theta: float, scaling: Mapping | Non
     return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
+def banded_frequencies(head_dim: int, theta: float, scaling: Mapping) -> torch.Tensor:
+    """64-bit ``f [D/2]`` of a rotary encoding whose long wavelengths are stretched (the rule of the Llama 3.1
+    models): with ``scaling = {factor, low, high, original}`` and a wavelength ``l = 2 pi / f``, ``f`` stays where ``l < original /
+    high``, becomes ``f / factor`` where ``l > original / low``, and between the two ``(1 - s) f / factor + s f`` with ``s =
+    (original / l - low) / (high - low)``."""
+    index = torch.arange(head_dim // 2, dtype=torch.float64)
+    freq = float(theta) ** (-2.0 * index / head_dim)
+    factor, low, high, original = (float(scaling[key]) for key in ("factor", "low", "high", "original"))
+    turns = original * freq / (2.0 * math.pi)  # original / l
+    if high > low:
+        blend = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+    else:
+        blend = (turns >= low).to(torch.float64)
+    return (1.0 - blend) * freq / factor + blend * freq
+
+
 def exact_rotary_tables(capacity: int, freq: torch.Tensor, magnitude: float) -> tuple[torch.Tensor, torch.Tensor]:
     """32-bit ``cos, sin [capacity, D/2]`` times ``magnitude`` from 64-bit angles ``pos * freq``, rounded once."""
     angles = torch.outer(torch.arange(capacity, dtype=torch.float64), freq)
@@ -64,7 +80,7 @@ def normed_store(runtime: Runtime, qkv, num_heads, num_kv_heads, head_dim, value
     gains of the projections' full sizes; ``ops.span_norm_store``, which rotates nothing).  ``values =
     {"keep": tensor}`` and/or ``{"blend": (tensor, weight)}``: the step's values as projected are left in
     ``keep``, and what is stored is mixed with ``blend`` (``ops.head_norm_store``).  ``shape``: what else the
-    per-head store takes (``normed``, ``norm_after``, ``values_are_keys``, ``query_temperature``, ``tail``)."""
+    per-head store takes (``normed``, ``norm_after``, ``values_are_keys``, ``query_temperature``, ``tail``, ``neighbours``)."""
     if span_norm is not None:
         if values or shape:
             raise ValueError("values are kept or mixed by the per-head store only")
@@ -99,8 +115,9 @@ class RotaryEncoding(PositionEncoding):
 
     ``interpolation = {factor, original, fast, slow}`` stretches the slow frequencies
     (:func:`interpolated_frequencies`); ``exact`` (implied by it) makes the tables from 64-bit angles
-    rounded once.  ``neighbours``: the pairs turned together are ``(2i, 2i + 1)``; only a part that
-    reads the tables itself (the latent layer's store) takes that.  ``head_dim`` may be smaller than the
+    rounded once, and so does ``bands = {factor, low, high, original}``
+    (:func:`banded_frequencies`).  ``neighbours``: the pairs turned together are ``(2i, 2i + 1)`` (the per-head
+    store and the latent layer's take that).  ``head_dim`` may be smaller than the
     heads it is applied to: their first ``head_dim`` elements are turned, the rest pass."""
 
     shareable = True
@@ -116,6 +133,7 @@ class RotaryEncoding(PositionEncoding):
         max_positions: int = 2048,
         initial_positions: int | None = None,
         interpolation: Mapping | None = None,
+        bands: Mapping | None = None,
         exact: bool = False,
         neighbours: bool = False,
     ) -> None:
@@ -126,7 +144,10 @@ class RotaryEncoding(PositionEncoding):
         self.theta = float(theta)
         self.scaling_factor = float(scaling_factor)
         self.interpolation = None if interpolation is None else dict(interpolation)
-        self.exact = bool(exact) or interpolation is not None
+        self.bands = None if bands is None else dict(bands)
+        if self.bands is not None and self.interpolation is not None:
+            raise ValueError("a rotary encoding's frequencies are stretched by one rule")
+        self.exact = bool(exact) or interpolation is not None or bands is not None
         self.neighbours = bool(neighbours)
         if self.exact and self.scaling_factor != 1.0:
             raise ValueError("positions divided by a factor and exact or interpolated tables exclude each other")
@@ -146,7 +167,11 @@ class RotaryEncoding(PositionEncoding):
             return
         target = max(num_positions, 2 * self.capacity, self.initial_capacity, 16)
         if self.exact:
-            cos, sin = exact_rotary_tables(target, *interpolated_frequencies(self.head_dim, self.theta, self.interpolation))
+            if self.bands is not None:
+                freq, magnitude = banded_frequencies(self.head_dim, self.theta, self.bands), 1.0
+            else:
+                freq, magnitude = interpolated_frequencies(self.head_dim, self.theta, self.interpolation)
+            cos, sin = exact_rotary_tables(target, freq, magnitude)
         else:
             cos, sin = rotary_tables(target, self.head_dim, self.theta, self.scaling_factor)
         if self.cos is not None:
@@ -159,13 +184,13 @@ class RotaryEncoding(PositionEncoding):
                          value_dim: int | None = None, head_norm: tuple | None = None, span_norm: tuple | None = None,
                          values: Mapping | None = None, shape: Mapping | None = None):
         if self.neighbours:
-            raise ValueError("the stores of whole heads turn the pairs (i, i + D/2) only")
+            shape = {**(shape or {}), "neighbours": True}  # (the per-head store turns them)
         if self.head_dim > head_dim:
             raise ValueError(f"{self.head_dim} turned elements do not fit heads of {head_dim}")
         self.ensure_capacity(ctx.max_context_len)
         slots = ctx.slot_mapping[cache.group] if cache.writable else None
         # (Tables narrower than the heads turn the heads' first elements only: the per-head store takes that.)
-        if (head_norm is not None or span_norm is not None or values or shape or self.head_dim != head_dim
+        if (head_norm is not None or span_norm is not None or values or shape or self.head_dim != head_dim or num_kv_heads == 0
                 or (value_dim is not None and value_dim != head_dim)):
             return normed_store(self.runtime, qkv, num_heads, num_kv_heads, head_dim, value_dim or head_dim, ctx, cache,
                                 slots, head_norm, self.cos, self.sin, span_norm, values, shape)
@@ -188,7 +213,8 @@ class NoPositionEncoding(PositionEncoding):
                          value_dim: int | None = None, head_norm: tuple | None = None, span_norm: tuple | None = None,
                          values: Mapping | None = None, shape: Mapping | None = None):
         slots = ctx.slot_mapping[cache.group] if cache.writable else None
-        if head_norm is not None or span_norm is not None or values or shape or (value_dim is not None and value_dim != head_dim):
+        if (head_norm is not None or span_norm is not None or values or shape or num_kv_heads == 0
+                or (value_dim is not None and value_dim != head_dim)):
             return normed_store(self.runtime, qkv, num_heads, num_kv_heads, head_dim, value_dim or head_dim, ctx, cache,
                                 slots, head_norm, None, None, span_norm, values, shape)
         return self.runtime.ops.rope_store(
