@@ -33,7 +33,7 @@ and one 2,048-token prompt), ``--shape 32b --batch 64 --fill-hbm`` (a cache pool
 free memory), ``--closed-loop C [--sampled]`` (the reference's serving profile driven offline: 256
 requests of 128..1,024 tokens in and 64..512 out, C in flight; the library's products run at a
 few step sizes that are all timed at start-up, about 70 s the first time), ``--attention-prefill T[,CTX]`` (the
-prefill attention kernel alone), ``--sample-kernel ROWS`` (the sampling kernel alone), ``--hbm-read`` (a kernel that only reads: what the memory gives), ``--only-prefill [TOKENS]`` (one prompt's prefill alone, 2,048 tokens or TOKENS), ``--designs [2k,4k]`` (the Sisisun design beside a Qwen2 model of equal layer sizes: prefill and decode; with ``--design kisadra`` the Kisadra design beside Sisisun, with ``--design dovudra`` the Dovudra design beside Kisadra, with ``--design legavik`` the Legavik design beside Kisadra), ``--kernel-shares TRACE.csv`` (no GPU: the per-kernel table of a
+prefill attention kernel alone), ``--sample-kernel ROWS`` (the sampling kernel alone), ``--hbm-read`` (a kernel that only reads: what the memory gives), ``--only-prefill [TOKENS]`` (one prompt's prefill alone, 2,048 tokens or TOKENS), ``--designs [2k,4k]`` (the Sisisun design beside a Qwen2 model of equal layer sizes: prefill and decode; with ``--design kisadra`` the Kisadra design beside Sisisun, with ``--design dovudra`` the Dovudra design beside Kisadra, with ``--design legavik`` the Legavik design beside Kisadra, with ``--design lukelix`` the Lukelix design beside Kisadra), ``--kernel-shares TRACE.csv`` (no GPU: the per-kernel table of a
 ``rocprofv3 --kernel-trace`` of any of these runs).
 """
 
@@ -124,9 +124,9 @@ def parse_args(argv: list[str] | None = None) -> argparse.Namespace:
                    help="prefill and decode of the Sisisun design (random weights) at layer sizes that resemble a real "
                         "model's (2k, 4k: the width), beside a Qwen2 model of the same width, heads, feed-forward and "
                         "number of layer runs; prints one JSON object and exits")
-    p.add_argument("--design", choices=["sisisun", "kisadra", "dovudra", "legavik"], default="sisisun",
+    p.add_argument("--design", choices=["sisisun", "kisadra", "dovudra", "legavik", "lukelix"], default="sisisun",
                    help="which design --designs measures: sisisun beside Qwen2, kisadra beside sisisun, dovudra beside kisadra, "
-                        "or legavik beside kisadra")
+                        "legavik beside kisadra, or lukelix beside kisadra")
     return p.parse_args(argv)
 
 
@@ -576,6 +576,32 @@ def legavik_pair(size: str) -> tuple[dict, dict]:
     return legavik, kisadra
 
 
+#: ``--designs --design lukelix``: the Lukelix configuration of a size (twelve layers: three of convolved attention, the
+#: last of which reads the first one's keys and values, each with a feed-forward, and nine of Mamba-2 without one) beside
+#: a Kisadra configuration of the same order: attention over one chunk longer than the prompt with a gated feed-forward two
+#: thirds as wide, gated linear attention without one in as many heads as give a layer the same parameters.
+def lukelix_pair(size: str) -> tuple[dict, dict]:
+    width, heads, kv, ff, states, gla_heads = {"2k": (2048, 16, 4, 8192, 64, 22), "4k": (4096, 32, 8, 14336, 128, 42)}[size]
+    turning = {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 1024}}
+    attention = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "conv": 4, "rot": turning}
+    state = {"heads": states, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    order = ["attention", "mamba2", "mamba2", "mamba2"] * 3
+    layers, beside = [], []
+    for index, kind in enumerate(order):
+        if kind == "attention":
+            layers.append({"type": kind, "mixer": dict(attention, kv_from=0) if index == 8 else attention, "mlp": {"kind": "dense", "ff": ff}})
+            beside.append({"type": kind, "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                   "mask": {"size": 1 << 20}}, "mlp": {"kind": "dense", "ff": ff * 2 // 3 // 64 * 64}})
+        else:
+            layers.append({"type": kind, "mixer": state, "mlp": None})
+            beside.append({"type": "gla", "mixer": {"heads": gla_heads, "dim": 128, "vdim": 128, "tau": 16.0, "rank": 16}, "mlp": None})
+    lukelix = {"architecture": "Lukelix", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "layers": layers,
+               "embedding": {"bigram": {"buckets": 32749, "mul_prev": 31, "mul_cur": 17}}}
+    kisadra = {"architecture": "Kisadra", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "layers": beside,
+               "loop": {"start": 0, "stop": 0, "times": 1}}
+    return lukelix, kisadra
+
+
 def mixer_work(mixer, batch: int, context: int, prompt: int) -> tuple[float, float]:
     """``(elements a decode step of `batch` requests at `context` tokens reads from the cache or state,
     multiply-adds x 2 of a prompt of `prompt` tokens inside the mixer beside its plain projections)``."""
@@ -588,6 +614,9 @@ def mixer_work(mixer, batch: int, context: int, prompt: int) -> tuple[float, flo
         # the decay, two reads and a write of the state, 2 flops each.
         state = mixer.num_heads * mixer.head_dim * mixer.value_dim
         return batch * (2 * state * 2.0 + 4.0 * (mixer.taps - 1) * mixer.channels), 8.0 * prompt * state
+    if kind == "Mamba2":
+        state = mixer.num_heads * mixer.state_dim * mixer.value_dim
+        return batch * (2 * state * 2.0 + 4.0 * (mixer.taps - 1) * mixer.channels), 4.0 * prompt * state
     if kind == "GatedLinearAttention":
         state = mixer.num_heads * mixer.head_dim * mixer.value_dim
         return batch * 2 * state * 2.0, 4.0 * prompt * state  # 32-bit state read and written: 2 x 2 run-dtype elements
@@ -642,7 +671,7 @@ def run_designs(sizes: list[str], dtype_name: str, steps: int, warmup: int, desi
     for size in sizes:
         size, _, only = size.partition(":")  # "2k:qwen2": that design alone; "2k:qwen2:prefill": that phase alone (for profiles)
         only, _, phase = only.partition(":")
-        labels, pair = {"legavik": (("legavik", "kisadra"), legavik_pair),
+        labels, pair = {"lukelix": (("lukelix", "kisadra"), lukelix_pair), "legavik": (("legavik", "kisadra"), legavik_pair),
                         "dovudra": (("dovudra", "kisadra"), dovudra_pair), "kisadra": (("kisadra", "sisisun"), kisadra_pair),
                         "sisisun": (("sisisun", "qwen2"), lambda s: design_pair(s))}[design]
         pair = pair(size)

@@ -1,0 +1,689 @@
+"""Lukelix on the GPU against the plain implementation (``tests/plain/lukelix_plain.py``): each mechanism
+alone (its kernel, and a one-layer model of it), whole prompts, every way of cutting requests into steps
+on so few pages and slots that they are used again, keys far back, at page borders and at a sequence's first
+positions through a layer's own keys and through another's, state that has to last, and greedy generation
+through the engine's own entry point."""
+
+from __future__ import annotations
+
+import json
+import random
+import subprocess
+import sys
+from pathlib import Path
+
+import pytest
+import torch
+
+import lukelix_tiny as lt
+import trace_helpers as th
+from plain import lukelix_plain as plain
+
+pytestmark = pytest.mark.gpu
+
+DEV = "cuda:0"
+ROOT = Path(__file__).resolve().parent.parent
+#: How far a position's logits may be off, relative to its largest (at least 1): the engine's 32-bit runs and its bfloat16
+#: runs (weights stored in bfloat16) against the plain implementation in 64-bit on the same weights ...
+FLOOR = {"float32": 1e-4, "bfloat16": 4e-2}
+#: ... or this many times what changing every weight by a relative error of the run's rounding does to that position, where
+#: that is more: a norm behind a part makes a position whose output is small against its terms (a head's key, a part of a
+#: gated norm) answer rounding ten times as strongly as others do.
+ANSWER = 4.0
+ROUNDING = {"float32": 2.0 ** -22, "bfloat16": 2.0 ** -9}
+
+
+@pytest.fixture(scope="module")
+def ops():
+    from turboserve_amd.kernels.ops import Ops
+
+    return Ops(DEV)
+
+
+def expect(folder, tokens: list[int], dtype: str) -> tuple[torch.Tensor, torch.Tensor]:
+    """The plain implementation's logits ``[T, V]`` in 64-bit and each position's bound ``[T]``."""
+    raw, tensors = lt.read_model_dir(folder)
+    tensors = {name: t.double() for name, t in tensors.items()}
+    want = plain.forward(raw, tensors, tokens)
+    scale = want.abs().amax(dim=-1).clamp_min(1.0)
+    bound = FLOOR[dtype] * scale
+    for seed in (1, 2):
+        g = torch.Generator().manual_seed(seed)
+        off = {name: t * (1.0 + ROUNDING[dtype] * torch.randn(t.shape, generator=g).double()) for name, t in tensors.items()}
+        bound = torch.maximum(bound, ANSWER * (plain.forward(raw, off, tokens) - want).abs().amax(dim=-1))
+    return want, bound
+
+
+def excess(got: torch.Tensor, expected: tuple[torch.Tensor, torch.Tensor]) -> float:
+    """The largest multiple of its bound that a position is off by."""
+    want, bound = expected
+    return float(((got.double() - want).abs().amax(dim=-1) / bound).max())
+
+
+def tokens_of(vocab: int, length: int, seed: int) -> list[int]:
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, vocab, (length,), generator=g).tolist()
+
+
+def stored_as(dtype: str) -> torch.dtype:
+    return torch.float32 if dtype == "float32" else torch.bfloat16
+
+
+def run_trace(folder, dtype: str, page: int, steps: list[dict], max_tokens: int | None = None, max_live: int = 4):
+    from turboserve_amd.engine.replay import TraceReplayer
+
+    replayer = TraceReplayer(folder, dtype=dtype, max_tokens=max_tokens or th.peak_tokens(steps, rounding=page),
+                             page_size=page, max_live=max_live)
+    outputs = {}
+    for record in steps:
+        logits = replayer.run_step(record)
+        if logits.shape[0]:
+            outputs[record["step"]] = logits.float().cpu()
+    replayer.manager.check_invariants()
+    assert all(pool.num_in_use == 0 for pool in replayer.manager.pools), "pages were not given back"
+    return outputs
+
+
+def near(got: torch.Tensor, want: torch.Tensor, dtype: torch.dtype, loose: float = 1.0) -> None:
+    tol = (2e-5 if dtype == torch.float32 else 1.6e-2) * loose
+    scale = float(want.abs().max().clamp_min(1e-3))
+    assert float((got.float().cpu() - want).abs().max()) <= tol * scale, float((got.float().cpu() - want).abs().max()) / scale
+
+
+# ---------------------------------------------------------------------------------------------
+# mechanisms alone: kernels
+# ---------------------------------------------------------------------------------------------
+
+
+def ints(values):
+    return torch.tensor(values, dtype=torch.int32, device=DEV)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("hidden,tokens", [(51, 5), (64, 70), (321, 7), (1000, 3), (2048, 70), (4096, 2), (5001, 2), (9000, 3)])
+def test_the_layer_norm_carries_the_residual_sum(ops, dtype, hidden, tokens):
+    """Every combination of a norm on the pending output and one on the sum, of a dense pending output and
+    partial sums (more of them than are in flight at a time) and none, of all rows and chosen ones."""
+    g = torch.Generator().manual_seed(hidden)
+    residual = 3.0 + torch.randn(tokens, hidden, generator=g)
+    tensors = {}
+    for name in ("post", "own"):
+        tensors[name] = (1 + 0.3 * torch.randn(hidden, generator=g)).to(dtype)
+        tensors[name + ".b"] = (0.2 * torch.randn(hidden, generator=g)).to(dtype)
+    wide = {name: t.float() for name, t in tensors.items()}
+    on = {name: t.to(DEV) for name, t in tensors.items()}
+    for splits in (None, 0, 1, 11):
+        pending = given = None
+        if splits is not None:
+            pending = 5.0 + torch.randn(max(splits, 1), tokens, hidden, generator=g)
+            given = pending.to(DEV) if splits else pending[0].to(dtype).to(DEV)
+            pending = pending.sum(0) if splits else pending[0].to(dtype).float()
+        for post in (False, True) if pending is not None else (False,):
+            for own in (False, True):
+                total = residual.clone()
+                if pending is not None:
+                    total = total + (0.7 * plain.layer_norm(pending, wide, "post", 1e-5) if post else pending)
+                want = plain.layer_norm(total, wide, "own", 1e-4) if own else total
+                rule = {"pending_norm": (on["post"], on["post.b"], 1e-5, 0.7) if post else None,
+                        "norm": (on["own"], on["own.b"], 1e-4) if own else None}
+                stream = residual.clone().to(DEV)
+                near(ops.add_layer_norm(stream, given, dtype, **rule), want, dtype)
+                near(stream, total, torch.float32)
+                stream = residual.clone().to(DEV)
+                near(ops.add_layer_norm(stream, given, dtype, ints([tokens - 1, 0, tokens - 1]), **rule), want[[tokens - 1, 0, tokens - 1]], dtype)
+                assert torch.equal(stream.cpu(), residual)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("hidden,buckets,mul_prev,mul_cur", [(52, 31, 7, 5), (64, 1, 3, 3), (33, 1009, 2**40 + 17, 12345678901), (320, 50, 0, 1)])
+def test_the_two_table_embedding_carries_the_last_token(ops, dtype, hidden, buckets, mul_prev, mul_cur):
+    """Three requests in portions of one to seven tokens, in turn and left out, through slots not in row order."""
+    g = torch.Generator().manual_seed(buckets)
+    vocab, lengths, slots = 90, [20, 1, 33], [2, 0, 3]
+    table, pairs = torch.randn(vocab, hidden, generator=g).to(dtype), torch.randn(buckets + 1, hidden, generator=g).to(dtype)
+    requests = [tokens_of(vocab, n, 10 + n) for n in lengths]
+    config = {"embedding": {"bigram": {"buckets": buckets, "mul_prev": mul_prev, "mul_cur": mul_cur}}}
+    want = [plain.embedding(config, {"embed": table.float(), "bigram": pairs.float()}, tokens) for tokens in requests]
+    held = torch.full((5, 1), 77, dtype=torch.int32, device=DEV)
+    held[slots] = 0
+    done, turn = [0] * 3, 0
+    got = [torch.zeros(n, hidden) for n in lengths]
+    while any(d < n for d, n in zip(done, lengths)):
+        live = [i for i in range(3) if done[i] < lengths[i] and (i + turn) % 4 != 0]
+        turn += 1
+        if not live:
+            continue
+        counts = {i: 1 if turn % 3 == 0 else min((1, 2, 7, 3)[(turn + i) % 4], lengths[i] - done[i]) for i in live}
+        ids = [t for i in live for t in requests[i][done[i]:done[i] + counts[i]]]
+        starts = [0]
+        for i in live:
+            starts.append(starts[-1] + counts[i])
+        out = ops.embed_bigram(table.to(DEV), pairs.to(DEV), ints(ids), held, ints([slots[i] for i in live]),
+                               ints([j for j, i in enumerate(live) for _ in range(counts[i])]), ints(starts), num_seqs=len(live),
+                               mul_prev=mul_prev, mul_cur=mul_cur).cpu()
+        for j, i in enumerate(live):
+            got[i][done[i]:done[i] + counts[i]] = out[starts[j]:starts[j + 1]]
+            done[i] += counts[i]
+    for one, other in zip(got, want):
+        near(one, other, torch.float32)
+    assert held.flatten().tolist() == [requests[1][-1] + 1, 77, requests[0][-1] + 1, requests[2][-1] + 1, 77]
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("taps,channels,silu,bias", [(1, 20, True, True), (2, 64, False, True), (3, 32, False, False), (4, 300, True, True),
+                                                     (5, 7, True, True), (8, 48, False, True)])
+def test_the_short_convolution_with_a_bias(ops, dtype, taps, channels, silu, bias):
+    """Portions long enough for the kernel that takes several rows a thread: requests that begin and end inside
+    its tiles, shorter than the taps, and one that goes on in a second step."""
+    g = torch.Generator().manual_seed(taps * 100 + channels)
+    lengths, slots, width, first = [19, 2, 1, 33, 8, 3], [4, 0, 6, 2, 1, 5], channels + 12, 4
+    weight = (0.6 * torch.randn(channels, taps, generator=g)).to(dtype)
+    add = (0.5 * torch.randn(channels, generator=g)).to(dtype) if bias else None
+    rows = [torch.randn(n + 5, width, generator=g).to(dtype).float() for n in lengths]
+    state = torch.full((8, max(taps - 1, 1), channels), float("nan"), device=DEV)
+    state[slots] = 0.0
+    done = [0] * len(lengths)
+    for counts in (lengths, [5] * len(lengths)):
+        proj = torch.cat([r[d:d + n] for r, d, n in zip(rows, done, counts)])
+        starts = [0]
+        for n in counts:
+            starts.append(starts[-1] + n)
+        out = ops.short_conv(proj.to(dtype).to(DEV), first, weight.to(DEV), state, ints(slots),
+                             ints([j for j, n in enumerate(counts) for _ in range(n)]), ints(starts), tokens=proj.shape[0],
+                             num_seqs=len(counts), dtype=dtype, silu=silu, bias=None if add is None else add.to(DEV))
+        for i, n in enumerate(counts):
+            y = plain.short_conv(rows[i][:, first:first + channels], weight.float())[done[i]:done[i] + n] + (0 if add is None else add.float())
+            near(out[starts[i]:starts[i + 1]], torch.nn.functional.silu(y) if silu else y, dtype)
+            done[i] += n
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,turned,tokens", [(4, 2, 16, 24, 8, 40), (3, 3, 12, 12, 12, 5), (2, 1, 128, 128, 128, 70),
+                                                                   (1, 1, 64, 32, 6, 33), (6, 0, 32, 32, 16, 90), (3, 0, 20, 20, 4, 2), (2, 2, 72, 40, 40, 37)])
+def test_the_store_turns_neighbouring_pairs(ops, dtype, heads, kv_heads, dim, vdim, turned, tokens):
+    """Norm, rotation of neighbouring pairs of a head's first elements, store; with key heads and with queries only,
+    in prompts and in steps of few tokens."""
+    g = torch.Generator().manual_seed(dim + tokens)
+    page, first = 8, 29
+    proj = torch.randn(tokens, (heads + kv_heads) * dim + kv_heads * vdim, generator=g).to(dtype)
+    gains = [(1 + 0.3 * torch.randn(dim, generator=g)).to(dtype) for _ in range(2)]
+    rot = {"base": 70.0, "dims": turned}
+    angles = torch.outer(torch.arange(first + tokens, dtype=torch.float64), torch.tensor(plain.frequencies(rot), dtype=torch.float64))
+    wide = proj.float()
+    padded = torch.cat([torch.zeros(first, wide.shape[1]), wide])
+
+    def turn(columns, count, gain):
+        x = plain.unit_rms(padded[:, columns:columns + count * dim].view(-1, count, dim), 1e-5) * gain.float()
+        return plain.turn_neighbours(x, rot)[first:]
+
+    pages = -(-(first + tokens) // page)
+    order = torch.randperm(pages, generator=g)
+    slots = torch.tensor([int(order[p // page]) * page + p % page for p in range(first, first + tokens)])
+    k_pages = torch.zeros(pages, max(kv_heads, 1), page, dim, dtype=dtype, device=DEV)
+    v_pages = torch.zeros(pages, max(kv_heads, 1), vdim, page, dtype=dtype, device=DEV)
+    q, stride = ops.head_norm_store(
+        proj.clone().to(DEV), k_pages if kv_heads else None, v_pages if kv_heads else None, gains[0].to(DEV), gains[1].to(DEV) if kv_heads else None,
+        1e-5, torch.arange(first, first + tokens, dtype=torch.int32, device=DEV), slots.to(torch.int32).to(DEV) if kv_heads else None,
+        heads, kv_heads, dim, vdim, page, dtype, cos=angles.cos().float().to(DEV), sin=angles.sin().float().to(DEV),
+        max_position=first + tokens - 1, neighbours=True)
+    near(q.flatten()[:].view(tokens, -1)[:, :heads * dim] if stride == q.shape[1] else q, turn(0, heads, gains[0]).reshape(tokens, -1), dtype)
+    if kv_heads:
+        near(k_pages[slots // page, :, slots % page], turn(heads * dim, kv_heads, gains[1]), dtype)
+        values = wide[:, (heads + kv_heads) * dim:].view(tokens, kv_heads, vdim)
+        near(v_pages[slots // page, :, :, slots % page], values, dtype)
+
+
+def plain_selective(u, d, t, heads, groups, n, p):
+    T, inner = u.shape[0], heads * p
+    x, B, C = u[:, :inner].view(T, heads, p), u[:, inner:inner + groups * n].view(T, groups, n), u[:, inner + groups * n:].view(T, groups, n)
+    dt = torch.nn.functional.softplus(d + t["dt_bias"].double(), threshold=50.0)
+    y = torch.zeros(T, heads, p, dtype=torch.float64)
+    for h in range(heads):
+        g = h // (heads // groups)
+        y[:, h] = plain.selective_walk(x[:, h], B[:, g], C[:, g], dt[:, h], float(t["a_log"][h].double().exp()), float(t["skip"][h]))
+    return y.reshape(T, inner)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("heads,groups,n,p,rates", [(4, 2, 24, 16, "mixed"), (1, 1, 1, 7, "mixed"), (3, 3, 33, 70, "slow"), (6, 2, 64, 64, "mixed"),
+                                                    (2, 1, 128, 48, "fast"), (4, 4, 136, 8, "slow"), (2, 2, 256, 72, "mixed"), (2, 1, 300, 20, "mixed"),
+                                                    (8, 1, 48, 40, "mixed")])
+def test_the_selective_state_whole_in_pieces_and_walked(ops, dtype, heads, groups, n, p, rates):
+    """Three requests side by side through slots not in row order: long portions (cut into pieces on the matrix
+    cores where the run and the sizes allow it: pieces that are full, one token over, one short), short ones, single
+    tokens.  The inputs are what the run's type holds, so even in bfloat16 runs the result is good to 32-bit: decays of
+    hundreds of tokens, of a few, and so strong that a token forgets all before it."""
+    g = torch.Generator().manual_seed(heads * 1000 + n)
+    lengths, slots, at = [300, 129, 31], [3, 1, 4], 3
+    shift = {"slow": -6.0, "mixed": -2.0, "fast": 3.0}[rates]
+    t = {"dt_bias": -1 + torch.randn(heads, generator=g), "a_log": shift + 1.5 * torch.randn(heads, generator=g), "skip": torch.randn(heads, generator=g)}
+    us = [torch.randn(m, heads * p + 2 * groups * n, generator=g).to(dtype) for m in lengths]
+    ds = [(2 * torch.randn(m, at + heads + 2, generator=g)).to(dtype) for m in lengths]
+    want = [plain_selective(u.double(), d[:, at:at + heads].double(), t, heads, groups, n, p).float() for u, d in zip(us, ds)]
+    on = {k: v.to(DEV) for k, v in t.items()}
+    pieces = ops.selective_pieces_supported(dtype, n, p)
+    assert pieces == (dtype == torch.bfloat16 and (n, p) in ((24, 16), (64, 64), (128, 48), (136, 8), (256, 72), (48, 40)))
+    for sizes in ([1000], [128, 60, 2, 40, 1], [257, 3]):
+        state = torch.full((6, heads, p, n), float("nan"), device=DEV)
+        state[slots] = 0.0
+        done, got, turn = [0] * 3, [torch.zeros_like(w) for w in want], 0
+        while any(d < m for d, m in zip(done, lengths)):
+            counts = {i: min(sizes[(turn + i) % len(sizes)], lengths[i] - done[i]) for i in range(3) if done[i] < lengths[i]}
+            turn += 1
+            live = sorted(counts, key=lambda i: counts[i] == 1)  # portions first, single tokens behind them
+            long = sum(1 for i in live if counts[i] > 1)
+            u = torch.cat([us[i][done[i]:done[i] + counts[i]] for i in live]).contiguous().to(DEV)
+            proj = torch.cat([ds[i][done[i]:done[i] + counts[i]] for i in live])
+            given = torch.stack([0.5 * proj.float(), 0.25 * proj.float(), 0.25 * proj.float()]).to(DEV) if turn % 2 else proj.to(DEV)
+            starts = [0]
+            for i in live:
+                starts.append(starts[-1] + counts[i])
+            plan = None
+            if pieces and long and turn % 3:
+                cut, carries = ops.linear_state_pieces([counts[i] for i in live[:long]], ops.selective_piece)
+                plan = (ops.device_ints(cut), ops.device_ints(carries), len(cut), len(carries))
+            y = ops.selective_state(u, given, at, on["dt_bias"], on["a_log"], on["skip"], state, ints([slots[i] for i in live]), ints(starts),
+                                    num_seqs=len(live), heads=heads, groups=groups, state_dim=n, value_dim=p, dtype=dtype, plan=plan).cpu()
+            for j, i in enumerate(live):
+                got[i][done[i]:done[i] + counts[i]] = y[starts[j]:starts[j + 1]]
+                done[i] += counts[i]
+        for one, other in zip(got, want):
+            near(one, other, torch.float32)
+        assert torch.isnan(state[[0, 2, 5]]).all()
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("width,parts,tokens", [(12, 3, 5), (64, 1, 70), (4096, 8, 3), (4096, 1, 3), (2050, 2, 4), (1500, 1, 300), (8192, 1, 260)])
+def test_the_gated_norm_in_parts(ops, dtype, width, parts, tokens):
+    g = torch.Generator().manual_seed(width + parts)
+    y, at = torch.randn(tokens, width, generator=g), 4
+    proj = (2 * torch.randn(tokens, width + 9, generator=g)).to(dtype)
+    gain = (1 + 0.3 * torch.randn(width, generator=g)).to(dtype)
+    want = plain.gated_group_norm(y, proj.float()[:, at:at + width], gain.float(), parts, 1e-5)
+    near(ops.gated_group_norm(y.to(DEV), proj.to(DEV), at, gain.to(DEV), 1e-5, parts, dtype), want, dtype)
+    wider = torch.nn.functional.pad(proj, (0, 3)).float()
+    near(ops.gated_group_norm(y.to(DEV), torch.stack([0.1 * wider] * 10).to(DEV), at, gain.to(DEV), 1e-5, parts, dtype), want, dtype)
+
+
+def test_one_launch_clears_a_slot_in_every_state():
+    from turboserve_amd.cache.layout import CacheLayout
+    from turboserve_amd.cache.storage import CacheStorage
+    from turboserve_amd.parts.base import FixedState
+
+    needs = [FixedState((3, 5)), FixedState((1,), torch.int32), FixedState((2, 64, 128)), FixedState((4,), torch.bfloat16), FixedState((7,))]
+    storage = CacheStorage(CacheLayout.from_needs(needs, [None] * 5), [], 8, 40, torch.float32, DEV)
+    for state in storage.states:
+        state.fill_(3)
+    gone = [1, 40, *range(2, 37)]
+    storage.zero_state_slots(gone)
+    for state in storage.states:
+        flat = state.reshape(41, -1).float().cpu()
+        assert bool((flat[gone] == 0).all()) and bool((flat[[0, 37, 38, 39]] == 3).all())
+
+
+# ---------------------------------------------------------------------------------------------
+# mechanisms alone: models of one layer (two where one reads the other's keys)
+# ---------------------------------------------------------------------------------------------
+
+WAVES = (4.0, 1.0, 4.0, 32)
+ALONE = {
+    "attention": [lt.layer(lt.attention(4, 2, 16, conv=3, scale=0.4, rot=8, bands=WAVES, base=100.0))],
+    "attention_no_convolution": [lt.layer(lt.attention(2, 1, 16, rot=16, base=100.0))],
+    "attention_no_rotation": [lt.layer(lt.attention(3, 3, 12, conv=2, scale=0.6))],
+    "attention_one_head": [lt.layer(lt.attention(1, 1, 20, 28, conv=5, rot=20, bands=WAVES, base=50.0))],
+    "attention_matrix_cores": [lt.layer(lt.attention(4, 2, 32, conv=4, rot=32, bands=WAVES, base=100.0))],
+    "attention_matrix_cores_in_part": [lt.layer(lt.attention(8, 1, 64, conv=3, rot=24, base=300.0))],
+    "attention_other_values": [lt.layer(lt.attention(4, 2, 32, 64, conv=3, rot=32, base=100.0))],
+    "shared_keys": [lt.layer(lt.attention(4, 2, 16, conv=3, scale=0.4, rot=8, base=100.0)),
+                    lt.layer(lt.attention(4, 2, 16, conv=2, scale=0.5, rot=8, base=100.0, kv_from=0))],
+    "shared_keys_no_convolution": [lt.layer(lt.attention(6, 2, 32, rot=32, bands=WAVES)), lt.layer(lt.attention(6, 2, 32, rot=32, bands=WAVES, kv_from=0))],
+    "shared_keys_other_values": [lt.layer(lt.attention(2, 1, 24, 8, conv=4)), lt.layer(lt.attention(2, 1, 24, 8, conv=4, kv_from=0))],
+    "state": [lt.layer(lt.mamba2(4, 16, 24, 2, 4, 2))],
+    "state_one_head": [lt.layer(lt.mamba2(1, 12, 9, 1, 2, 1))],
+    "state_a_group_a_head": [lt.layer(lt.mamba2(3, 8, 40, 3, 3, 3))],
+    "state_one_tap": [lt.layer(lt.mamba2(2, 32, 16, 1, 1, 4))],
+    "state_wide": [lt.layer(lt.mamba2(2, 72, 136, 2, 4, 1))],
+    "feed_forward": [lt.layer(lt.attention(1, 1, 8, rot=4), 52)],
+    "state_feed_forward": [lt.layer(lt.mamba2(2, 8, 16, 1, 4, 1), 36)],
+}
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("which", sorted(ALONE))
+def test_one_layer_models(tmp_path, which, dtype):
+    """Whole, token by token from the start, and in portions, against the plain implementation."""
+    config = {"architecture": "Lukelix", "vocab": 61, "width": 40, "norm": {"eps": 1e-5}, "embedding": lt.bigram(23, 5, 3), "layers": ALONE[which]}
+    folder = lt.make_model_dir(tmp_path / "m", config, 31, stored_as(dtype), std=0.2)
+    requests = {"a": tokens_of(61, 140, 1), "b": tokens_of(61, 3, 2)}
+    want = {rid: expect(folder, tokens, dtype) for rid, tokens in requests.items()}
+    for steps in (th.whole(requests), th.prefix_then_single(requests, tail=139), th.portions(requests, (2, 5, 71, 3))):
+        got = th.collect(steps, run_trace(folder, dtype, 8, steps), requests)
+        for rid in requests:
+            assert excess(got[rid], want[rid]) <= 1.0, (which, rid)
+
+
+# ---------------------------------------------------------------------------------------------
+# whole models, every cutting
+# ---------------------------------------------------------------------------------------------
+
+
+@pytest.fixture(scope="module", params=sorted(lt.TINY))
+def case(request, tmp_path_factory):
+    config, seed, page = lt.TINY[request.param]
+    base = tmp_path_factory.mktemp(f"lukelix_{request.param}")
+    folders = {dtype: lt.make_model_dir(base / dtype, config, seed, stored_as(dtype)) for dtype in ("float32", "bfloat16")}
+    lengths = (1, 2, 37, 180, 70, 9)
+    requests = {f"r{i}": tokens_of(config["vocab"], n, 100 * seed + i) for i, n in enumerate(lengths)}
+    expected = {dtype: {rid: expect(folder, tokens, dtype) for rid, tokens in requests.items()} for dtype, folder in folders.items()}
+    return {"name": request.param, "page": page, "folders": folders, "requests": requests, "expected": expected}
+
+
+def check_against_plain(case, dtype: str, steps: list[dict], **more) -> None:
+    outputs = run_trace(case["folders"][dtype], dtype, case["page"], steps, **more)
+    got = th.collect(steps, outputs, case["requests"])
+    for rid, want in case["expected"][dtype].items():
+        worst = excess(got[rid], want)
+        assert worst <= 1.0, f"{case['name']} {dtype} {rid}: {worst:.2f} times the bound"
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_whole_prompts(case, dtype):
+    check_against_plain(case, dtype, th.whole(case["requests"]))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_prefix_then_token_by_token(case, dtype):
+    check_against_plain(case, dtype, th.prefix_then_single(case["requests"], tail=40))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("sizes", [(2, 3, 5, 2, 16, 7), (33, 2, 70, 64), (1, 2)])
+def test_portions_of_changing_size(case, dtype, sizes):
+    check_against_plain(case, dtype, th.portions(case["requests"], sizes))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_mixed_batches_on_pages_and_slots_that_are_used_again(case, dtype):
+    """Three requests live at a time out of six, on a pool sized for the peak and three state slots: every
+    page and slot serves several requests, and what one left there must not reach the next."""
+    steps = th.mixed(case["requests"], (7, 2, 19, 66, 3), max_live=3, decode_tail=9)
+    check_against_plain(case, dtype, steps, max_live=3)
+
+
+def test_long_decoding(case):
+    """One short prompt, then 180 tokens one by one (recorded steps), in 32-bit: state and last inputs are carried
+    through every one of them."""
+    config = lt.TINY[case["name"]][0]
+    tokens = tokens_of(config["vocab"], 186, 4242)
+    requests = {"long": tokens}
+    steps = th.prefix_then_single(requests, tail=180)
+    got = th.collect(steps, run_trace(case["folders"]["float32"], "float32", case["page"], steps), requests)["long"]
+    assert excess(got, expect(case["folders"]["float32"], tokens, "float32")) <= 1.0, case["name"]
+
+
+def test_cuttings_agree_in_32_bit(case):
+    """The logits of a position do not depend on how its request was cut or batched, beyond rounding."""
+    folder, page = case["folders"]["float32"], case["page"]
+    ways = {"whole": th.whole(case["requests"]), "single": th.prefix_then_single(case["requests"], tail=40),
+            "portions": th.portions(case["requests"], (2, 5, 3, 24)), "mixed": th.mixed(case["requests"], (5, 2, 21, 80), max_live=4)}
+    results = {name: th.collect(steps, run_trace(folder, "float32", page, steps), case["requests"]) for name, steps in ways.items()}
+    for name, got in results.items():
+        for rid, base in results["whole"].items():
+            scale = base.abs().amax(dim=-1, keepdim=True).clamp_min(1.0)
+            assert float(((got[rid] - base).abs() / scale).max()) <= 5e-5, (name, rid)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_the_replay_program(case, dtype, tmp_path):
+    """``bin/trace_run`` itself on a model folder of this design, steps that want nothing included."""
+    if case["name"] != "A":
+        pytest.skip("one configuration is enough for the subprocess test")
+    steps = th.mixed(case["requests"], (7, 2, 19, 66, 3), max_live=3, decode_tail=9)
+    for record in steps[1::3]:
+        for entry in record["entries"]:
+            entry["want"] = []
+    out = tmp_path / "out"
+    proc = subprocess.run(
+        [sys.executable, str(ROOT / "bin" / "trace_run"), "--model", str(case["folders"][dtype]), "--dtype", dtype,
+         "--out", str(out), "--max-tokens", str(th.peak_tokens(steps)), "--page-size", str(case["page"])],
+        input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=600,
+    )
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [line for line in proc.stdout.splitlines() if line.startswith("done ")] == [f"done {s['step']}" for s in steps]
+    import numpy as np
+
+    vocab = lt.TINY["A"][0]["vocab"]
+    position = {rid: 0 for rid in case["requests"]}
+    for record in steps:
+        wanted = sum(len(e["want"]) for e in record["entries"])
+        path = out / f"{record['step']}.f32"
+        assert path.exists() == bool(wanted)
+        got = torch.from_numpy(np.fromfile(path, dtype="<f4").reshape(wanted, vocab).copy()) if wanted else None
+        row = 0
+        for entry in record["entries"]:
+            for place in entry["want"]:
+                want, bound = (t[position[entry["id"]] + place][None] for t in case["expected"][dtype][entry["id"]])
+                assert excess(got[row:row + 1], (want, bound)) <= 1.0
+                row += 1
+            position[entry["id"]] += len(entry["tokens"])
+
+
+def random_config(rng: random.Random) -> dict:
+    layers: list[dict] = []
+    for index in range(rng.randint(1, 6)):
+        ff = rng.choice([None, None, 12, 44, 64])
+        sources = [i for i, one in enumerate(layers) if one["type"] == "attention" and "kv_from" not in one["mixer"]]
+        if rng.random() < 0.5:
+            heads_of = rng.choice([1, 2, 3, 4, 6])
+            groups = rng.choice([k for k in (1, 2, 3, 6) if heads_of % k == 0])
+            p = rng.choice([4, 8, 12, 16, 40, 64])
+            parts = rng.choice([k for k in (1, 2, 3, 4, 8) if heads_of * p % k == 0 and (k == 1 or heads_of * p // k >= 8)])
+            layers.append(lt.layer(lt.mamba2(heads_of, p, rng.choice([3, 8, 16, 20, 64, 96]), groups, rng.choice([1, 2, 3, 4, 5]), parts), ff))
+        elif sources and rng.random() < 0.6:
+            source = rng.choice(sources)
+            mixer = dict(layers[source]["mixer"], kv_from=source, scale=rng.choice([0.2, 0.5, 0.9]))
+            mixer.pop("conv", None)
+            if rng.random() < 0.7:
+                mixer["conv"] = rng.choice([1, 2, 3, 4])
+            layers.append({"type": "attention", "mixer": mixer, "mlp": None if ff is None else {"kind": "dense", "ff": ff}})
+        else:
+            kv, dim = rng.choice([1, 1, 2, 3]), rng.choice([8, 12, 16, 20, 32, 64])
+            bands = rng.choice([None, (rng.choice([2.0, 8.0, 40.0]), rng.choice([0.5, 1.0]), rng.choice([2.0, 4.0]), rng.choice([8, 64, 1024]))])
+            layers.append(lt.layer(lt.attention(kv * rng.choice([1, 2, 3, 4]), kv, dim, rng.choice([dim, dim, 8, 24, 40]),
+                                                conv=rng.choice([None, 1, 2, 3, 4]), scale=rng.choice([None, 0.2, 0.5]),
+                                                rot=rng.choice([None, 2, dim // 2, dim]), bands=bands, base=rng.choice([10.0, 1000.0, 1e6])), ff))
+    config = {"architecture": "Lukelix", "vocab": rng.choice([50, 97, 256]), "width": rng.choice([40, 51, 64, 72, 96, 100, 128]),
+              "norm": {"eps": rng.choice([1e-6, 1e-5])}, "layers": layers}
+    if rng.random() < 0.8:
+        config["embedding"] = lt.bigram(rng.choice([1, 17, 1000]), rng.choice([0, 1, 31, 10**9 + 7]), rng.choice([1, 17, 65537]))
+    return config
+
+
+@pytest.mark.parametrize("trial", range(10))
+def test_random_configurations_replay_like_plain(trial, tmp_path):
+    """Seeded random configurations: one to six layers of either mixer in any order, layers that read the keys of
+    any earlier one, rotation of two elements, half a head, a whole head or none, convolutions of one to five taps or
+    none, groups and equal parts of every number that divides; whole, token by token and mixed."""
+    rng = random.Random(7000 + trial)
+    config = random_config(rng)
+    lengths = [rng.randint(1, 6), rng.randint(10, 60), rng.randint(100, 200), rng.randint(20, 90)]
+    requests = {f"r{i}": [rng.randrange(config["vocab"]) for _ in range(n)] for i, n in enumerate(lengths)}
+    for dtype in ("float32", "bfloat16"):
+        folder = lt.make_model_dir(tmp_path / dtype, config, trial, stored_as(dtype))
+        want = {rid: expect(folder, tokens, dtype) for rid, tokens in requests.items()}
+        ways = (th.whole(requests), th.prefix_then_single(requests, tail=20),
+                th.mixed(requests, (7, 2, 40, 150, 3), max_live=4, decode_tail=5))
+        for steps in ways:
+            outputs = run_trace(folder, dtype, 16, steps, max_tokens=th.peak_tokens(steps))
+            got = th.collect(steps, outputs, requests)
+            for rid in requests:
+                assert excess(got[rid], want[rid]) <= 1.0, (trial, dtype, rid, config)
+
+
+# ---------------------------------------------------------------------------------------------
+# one key that a query rests on, through a layer's own keys and through another layer's: far back, at page
+# borders, at the first positions
+# ---------------------------------------------------------------------------------------------
+
+MARK, ASKS, OTHER = 7, 9, 11  # the token that is looked for, the token whose query looks for it, one that is neither
+
+
+def marked_model(folder, dtype: torch.dtype, shared: bool):
+    """An attention layer whose query of ``ASKS`` and key of ``MARK`` point the same way in the part of a head that is
+    not turned, with a scale under which that one score stands above all others, and a value of ``MARK`` that reaches the
+    logits.  No other token has anything in the two channels that make them; the convolutions pass the current
+    token on.  With ``shared`` the keys and values are an earlier layer's, whose own output is switched off."""
+    mixers = [lt.attention(2, 1, 16, conv=3, scale=1.5, rot=8, base=100.0)]
+    if shared:
+        mixers.append(lt.attention(2, 1, 16, conv=2, scale=1.5, rot=8, base=100.0, kv_from=0))
+    config = {"architecture": "Lukelix", "vocab": 40, "width": 32, "norm": {"eps": 1e-5}, "embedding": lt.bigram(13, 3, 5),
+              "layers": [lt.layer(mixer) for mixer in mixers]}
+    tensors = lt.draw_tensors(config, 5, torch.float32, 0.1)
+    tensors["embed"][:, :2] = 0.0
+    tensors["bigram"][:, :2] = 0.0
+    tensors["embed"][MARK, 0] = 3.0
+    tensors["embed"][ASKS, 1] = 3.0
+    towards = torch.zeros(16)
+    towards[8:] = torch.tensor([1.0, -1.0, 1.0, 1.0, -1.0, 1.0, -1.0, -1.0])
+    last = len(mixers) - 1
+    if shared:
+        tensors["l0.mix.o"][:] = 0.0
+        tensors["l0.norm1.b"][:2] = 0.0
+    tensors["l0.mix.k"][:, 0], tensors["l0.mix.k"][:, 1] = 6.0 * towards, 0.0
+    tensors["l0.mix.v"][:, 0] = 4.0 * torch.randn(16, generator=torch.Generator().manual_seed(3))
+    for head in range(2):
+        tensors[f"l{last}.mix.q"][16 * head:16 * head + 16, 1] = 6.0 * towards
+        tensors[f"l{last}.mix.q"][16 * head:16 * head + 16, 0] = 0.0
+    for name in tensors:
+        if name.endswith(".conv"):
+            tensors[name] *= 0.1
+            tensors[name][:, -1] = 1.0
+    tensors = {name: t.to(dtype).contiguous() for name, t in tensors.items()}
+    return lt.make_model_dir(folder, config, 0, tensors=tensors)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("shared", [False, True])
+@pytest.mark.parametrize("mark_at", [0, 1, 2, 15, 16, 17, 127, 128, 230])
+def test_a_key_far_back_is_found(tmp_path, dtype, shared, mark_at):
+    """The plain implementation says what the mark is worth at the last position; the engine agrees with it in
+    every cutting: whole, the last tokens one by one, portions."""
+    folder = marked_model(tmp_path / "m", stored_as(dtype), shared)
+    g = torch.Generator().manual_seed(mark_at)
+    tokens = [t if t not in (MARK, ASKS) else OTHER for t in torch.randint(0, 40, (260,), generator=g).tolist()]
+    tokens[-1], tokens[mark_at] = ASKS, MARK
+    raw, tensors = lt.read_model_dir(folder)
+    want, bound = expect(folder, tokens, dtype)
+    without = plain.forward(raw, tensors, [t if t != MARK else OTHER for t in tokens])
+    moved = float((want[-1] - without[-1]).abs().max() / want[-1].abs().max())
+    assert moved > 0.3, f"the mark moves the last logits by {moved:.3f}"
+    requests = {"m": tokens}
+    for steps in (th.whole(requests), th.prefix_then_single(requests, tail=12), th.portions(requests, (259, 1)), th.portions(requests, (5, 2, 16, 3))):
+        got = th.collect(steps, run_trace(folder, dtype, 16, steps), requests)["m"]
+        assert excess(got[-1:], (want[-1:], bound[-1:])) <= 1.0
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_what_a_token_left_in_the_state_hundreds_of_tokens_back_still_counts(tmp_path, dtype):
+    """A layer whose state hardly decays: a token 250 positions back changes the last logits, and the engine
+    follows it whole, token by token and in portions."""
+    config = {"architecture": "Lukelix", "vocab": 40, "width": 32, "norm": {"eps": 1e-5}, "embedding": lt.bigram(13, 3, 5),
+              "layers": [lt.layer(lt.mamba2(4, 16, 16, 2, 4, 2))]}
+    tensors = lt.draw_tensors(config, 8, torch.float32, 0.25)
+    tensors["l0.mix.A_log"][:] = -7.0
+    tensors["l0.mix.D"][:] = 0.0
+    tensors["embed"][MARK] *= 6.0
+    tensors = {name: t.to(stored_as(dtype)).contiguous() for name, t in tensors.items()}
+    folder = lt.make_model_dir(tmp_path / "m", config, 0, tensors=tensors)
+    raw, loaded = lt.read_model_dir(folder)
+    tokens = [t if t != MARK else OTHER for t in tokens_of(40, 260, 77)]
+    tokens[9] = MARK
+    want, bound = expect(folder, tokens, dtype)
+    other = plain.forward(raw, loaded, [t if t != MARK else OTHER for t in tokens])
+    moved = float((want[-1] - other[-1]).abs().max() / want[-1].abs().max())
+    assert moved > 0.05, f"the early token moves the last logits by {moved:.4f}"
+    requests = {"m": tokens}
+    for steps in (th.whole(requests), th.prefix_then_single(requests, tail=200), th.portions(requests, (9, 2, 64, 1, 130))):
+        got = th.collect(steps, run_trace(folder, dtype, 16, steps), requests)["m"]
+        assert excess(got, (want, bound)) <= 1.0
+
+
+# ---------------------------------------------------------------------------------------------
+# generation through the engine's own entry point and the command line
+# ---------------------------------------------------------------------------------------------
+
+
+@pytest.mark.parametrize("name,blocks", [("A", 40), ("B", 40), ("C", 40), ("A", 8)])
+def test_greedy_generation_through_the_engine(tmp_path, name, blocks):
+    """Twice on one engine, steps launched ahead (the token before the one that is fed is then known on the device
+    only); with few pages requests are preempted and run again from their first token."""
+    from turboserve_amd.config.engine_config import EngineConfig, SchedulerConfig
+    from turboserve_amd.engine.llm_engine import LLMEngine
+    from turboserve_amd.sampling.params import SamplingParams
+
+    config, seed, page = lt.TINY[name]
+    folder = lt.make_model_dir(tmp_path / "gen", config, seed + 5, torch.float32, std=0.2)
+    raw, tensors = lt.read_model_dir(folder)
+    prompts = [tokens_of(config["vocab"], n, 900 + n) for n in (3, 21, 1, 50)]
+    new = 40
+    want = [lt.greedy(raw, tensors, prompt, new) for prompt in prompts]
+    engine = LLMEngine(EngineConfig(
+        model=str(folder), dtype="float32",
+        scheduler=SchedulerConfig(max_num_seqs=4, max_num_batched_tokens=64, block_size=page, num_blocks=blocks),
+    ))
+    outputs = engine.generate(prompts, SamplingParams(max_tokens=new, temperature=0.0, ignore_eos=True))
+    assert [out.new_token_ids for out in outputs] == want
+    again = engine.generate(list(reversed(prompts)), SamplingParams(max_tokens=new, temperature=0.0, ignore_eos=True))
+    assert [out.new_token_ids for out in again] == list(reversed(want))
+
+
+def test_a_model_of_states_alone_is_served_without_pages(tmp_path):
+    """No layer keeps keys: the engine has state slots and no page pool, and requests end by their length."""
+    from turboserve_amd.config.engine_config import EngineConfig, SchedulerConfig
+    from turboserve_amd.engine.llm_engine import LLMEngine
+    from turboserve_amd.sampling.params import SamplingParams
+
+    config = {"architecture": "Lukelix", "vocab": 61, "width": 40, "norm": {"eps": 1e-5}, "embedding": lt.bigram(23, 5, 3),
+              "layers": [lt.layer(lt.mamba2(4, 16, 24, 2, 4, 2), 36), lt.layer(lt.mamba2(2, 32, 16, 1, 3, 1))]}
+    folder = lt.make_model_dir(tmp_path / "m", config, 3, torch.float32, std=0.2)
+    raw, tensors = lt.read_model_dir(folder)
+    prompts = [tokens_of(61, n, n) for n in (5, 70, 1)]
+    for blocks in (16, None):
+        engine = LLMEngine(EngineConfig(model=str(folder), dtype="float32", scheduler=SchedulerConfig(
+            max_num_seqs=2, max_num_batched_tokens=32, block_size=16, num_blocks=blocks)))
+        outputs = engine.generate(prompts, SamplingParams(max_tokens=12, temperature=0.0, ignore_eos=True))
+        assert [out.new_token_ids for out in outputs] == [lt.greedy(raw, tensors, prompt, 12) for prompt in prompts]
+
+
+def test_the_command_line_serves_the_design(tmp_path, capsys):
+    """``engine random-model`` writes a folder from a config.json of the design, ``engine generate``
+    completes prompts given as token ids with the plain implementation's greedy tokens, and ``engine
+    kv-size`` sizes a cache in which the layer that reads another's keys takes no pages."""
+    import re
+
+    from turboserve_amd import cli
+
+    config, _, page = lt.TINY["A"]
+    source = tmp_path / "config.json"
+    source.write_text(json.dumps(config))
+    folder = tmp_path / "model"
+    assert cli.main(["engine", "random-model", "--config", str(source), "--out", str(folder), "--seed", "4", "--dtype", "float32"]) == 0
+    raw, tensors = lt.read_model_dir(folder)
+    prompts = [tokens_of(config["vocab"], n, 600 + n) for n in (4, 19)]
+    capsys.readouterr()
+    args = ["engine", "generate", "--model", str(folder), "--dtype", "float32", "--max-tokens", "12", "--ignore-eos",
+            "--num-blocks", "24", "--block-size", str(page)]
+    assert cli.main(args + [a for p in prompts for a in ("--prompt-ids", ",".join(map(str, p)))]) == 0
+    shown = [json.loads(m) for m in re.findall(r"^output \d+: (\[.*\])$", capsys.readouterr().out, flags=re.M)]
+    assert len(shown) == len(prompts)
+    for prompt, got in zip(prompts, shown):
+        tokens = list(prompt)
+        for token in got:  # the written model's weights are small: equal logits are allowed for
+            logits = plain.forward(raw, tensors, tokens)[-1]
+            assert float(logits.max() - logits[token]) <= 1e-4 * float(logits.abs().max().clamp_min(1.0))
+            tokens.append(token)
+    assert cli.main(["engine", "kv-size", "--model", str(folder), "--dtype", "bfloat16", "--max-model-len", "64",
+                     "--block-size", str(page)]) == 0
+    sizing = capsys.readouterr().out
+    sizing = json.loads(sizing[sizing.index("{"):])
+    assert sizing["bytes_per_block"] == [2 * (16 + 24) * 2 * page] and sizing["activation_bytes"] > 0

@@ -11,6 +11,7 @@ The reference has one pool with the same block ids for every layer
 
 from __future__ import annotations
 
+import math
 from collections.abc import Sequence
 from dataclasses import dataclass
 
@@ -122,3 +123,7 @@ class CacheLayout:
 
     def bytes_per_token(self, itemsize: int) -> int:
         return sum(group.elements_per_token() for group in self.groups) * itemsize
+
+    def state_bytes_per_slot(self) -> int:
+        """Bytes a request's slot takes in the state tensors of all entries."""
+        return sum(math.prod(need.shape) * need.dtype.itemsize for _, need in self.state_entries)

@@ -1,7 +1,7 @@
 """How many cache pages to allocate (src/turboserve/engine/runtime/memory.py:172-381).
 
 An explicit page count wins; otherwise the pages fill what is left of the memory budget after
-the weights and an estimate of a step's activations; a ``max_model_len`` caps it at what
+the weights, the state tensors of layers that keep state and an estimate of a step's activations; a ``max_model_len`` caps it at what
 ``max_num_seqs`` requests of that length can use.  Windowed groups never need more than a
 window plus one portion per request, so they are sized to that and the rest goes to the
 groups that keep every key.
@@ -39,6 +39,7 @@ class CacheSizing:
     reason: str
     total_bytes: int | None = None
     free_bytes: int | None = None
+    state_bytes: int = 0  # the state tensors: a row per slot and the padding row
 
     def to_dict(self) -> dict[str, Any]:
         return asdict(self)
@@ -72,6 +73,7 @@ def size_cache(
     per_page = layout.bytes_per_page(page, itemsize)
     windows = layout.windows()
     kept = layout.kept()
+    state_bytes = layout.state_bytes_per_slot() * (scheduler.max_num_seqs + 1)
     cap = None if max_model_len is None else ceil_div(max_model_len, page) * scheduler.max_num_seqs
 
     def clamp(group: int, count: int) -> int:
@@ -86,13 +88,14 @@ def size_cache(
         counts = [clamp(g, scheduler.num_blocks) if windows[g] is not None else scheduler.num_blocks
                   for g in range(len(per_page))]
         return CacheSizing(counts, page, per_page, sum(c * b for c, b in zip(counts, per_page)),
-                           min(c * page for c in counts), None, activation_bytes, "explicit num_blocks")
+                           min((c * page for c in counts), default=0), None, activation_bytes, "explicit num_blocks",
+                           state_bytes=state_bytes)
     if memory is None:
         free, total = torch.cuda.mem_get_info(device)
     else:
         free, total = memory
     used = total - free
-    budget = int(total * gpu_memory_utilization) - used - activation_bytes
+    budget = int(total * gpu_memory_utilization) - used - activation_bytes - state_bytes
     counts = [0] * len(per_page)
     remaining = budget
     for g, window in enumerate(windows):
@@ -107,8 +110,8 @@ def size_cache(
     if remaining < 0 or any(c < 1 for c in counts):
         raise MemoryProfileError(
             f"no room for a cache page: budget {budget} bytes after {used} used and {activation_bytes} "
-            f"for activations; pages take {per_page} bytes"
+            f"for activations and {state_bytes} for state; pages take {per_page} bytes"
         )
     reason = "memory budget" if cap is None or any(counts[g] < cap for g in full) else "max_model_len cap"
     return CacheSizing(counts, page, per_page, sum(c * b for c, b in zip(counts, per_page)),
-                       min(c * page for c in counts), budget, activation_bytes, reason, total, free)
+                       min((c * page for c in counts), default=0), budget, activation_bytes, reason, total, free, state_bytes)

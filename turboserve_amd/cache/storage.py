@@ -53,6 +53,12 @@ class CacheStorage:
             torch.zeros((num_state_slots + 1, *need.shape), dtype=need.dtype, device=device)
             for _, need in layout.state_entries
         ]
+        #: On a GPU: address and row bytes of every state tensor, so that one launch clears a slot in all of them.
+        self._zero_table: torch.Tensor | None = None
+        row_bytes = [state[0].numel() * state.element_size() for state in self.states]
+        if self.states and self.states[0].is_cuda and all(count % 4 == 0 for count in row_bytes):
+            self._zero_table = torch.tensor([[state.data_ptr(), count] for state, count in zip(self.states, row_bytes)],
+                                            dtype=torch.int64).to(self.states[0].device)
 
     def num_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.tensors())
@@ -93,6 +99,13 @@ class CacheStorage:
     def zero_state_slots(self, slots: Sequence[int]) -> None:
         """Clear the state of freshly taken slots (a request starts from zero state)."""
         if not slots or not self.states:
+            return
+        if any(not 0 <= slot <= self.num_state_slots for slot in slots):
+            raise ValueError(f"state slots {list(slots)} are not all inside the {self.num_state_slots} slots")
+        if self._zero_table is not None:
+            from turboserve_amd.kernels.ops import zero_state_rows
+
+            zero_state_rows(self._zero_table, list(slots))
             return
         index = torch.tensor(list(slots), dtype=torch.long, device=self.states[0].device)
         for state in self.states:

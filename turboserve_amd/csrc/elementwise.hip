@@ -865,3 +865,37 @@ extern "C" int ts_activate(void* out, const void* x, int in_f32, int splits, lon
     return TS_ERR_DTYPE;
   return ts_launch_status();
 }
+
+// ---------------------------------------------------------------------------------------------
+// clearing the state of requests that start: rows `slots` of every state tensor, one launch
+// ---------------------------------------------------------------------------------------------
+#define ZERO_SLOTS 32
+
+struct ZeroSlots {
+  int at[ZERO_SLOTS];
+};
+
+// table [n][2]: a state tensor's address and the bytes of one of its rows (a multiple of 4).
+__global__ void __launch_bounds__(256) zero_state_rows_kernel(const long long* __restrict__ table, ZeroSlots slots) {
+  const size_t words = (size_t)table[2 * blockIdx.y + 1] / 4;
+  uint32_t* row = reinterpret_cast<uint32_t*>(table[2 * blockIdx.y]) + (size_t)slots.at[blockIdx.x] * words;
+  const size_t step = (size_t)gridDim.z * blockDim.x, from = (size_t)blockIdx.z * blockDim.x + threadIdx.x;
+  if (words % 4 == 0 && ((uintptr_t)row & 15) == 0) {
+    for (size_t i = from; i < words / 4; i += step) reinterpret_cast<uint4*>(row)[i] = make_uint4(0u, 0u, 0u, 0u);
+  } else {
+    for (size_t i = from; i < words; i += step) row[i] = 0u;
+  }
+}
+
+// `slots` is host memory.
+extern "C" int ts_zero_state_rows(const long long* table, int n, const int* slots, int count, hipStream_t stream) {
+  if (n == 0 || count == 0) return TS_OK;
+  if (!table || !slots || n < 0 || n > 65535 || count < 0) return TS_ERR_ARG;
+  for (int first = 0; first < count; first += ZERO_SLOTS) {
+    const int here = count - first < ZERO_SLOTS ? count - first : ZERO_SLOTS;
+    ZeroSlots some;
+    for (int i = 0; i < ZERO_SLOTS; ++i) some.at[i] = slots[first + (i < here ? i : 0)];
+    hipLaunchKernelGGL(zero_state_rows_kernel, dim3(here, n, 32), dim3(256), 0, stream, table, some);
+  }
+  return ts_launch_status();
+}

@@ -11,9 +11,9 @@
 // ts_short_conv computes every row of the step and leaves the state alone; ts_short_conv_carry, launched
 // behind it, moves each request's last K - 1 inputs into its slot.  In a step whose requests all bring one
 // token (`single`), the thread that computes a channel of a request also moves the channel's state on, and
-// nothing is launched behind it.  Prompt portions in bfloat16 take four channels a thread with 8-byte
-// accesses (short_conv_rows_kernel), the same arithmetic.
-#include "common.hpp"
+// nothing is launched behind it.  Prompt portions in bfloat16 take four channels by eight rows a thread
+// (short_conv_rows_kernel), the same arithmetic.
+#include "vec.hpp"
 
 template <typename P>
 __device__ __forceinline__ float sc_input(const P* p, int splits, size_t stride) {
@@ -65,66 +65,65 @@ short_conv_kernel(O* __restrict__ out, const P* __restrict__ proj, int splits, s
   out[(size_t)t * channels + c] = from_float<O>(y);
 }
 
-// Prompt portions: bfloat16 in, four neighbouring channels a thread, 8-byte loads of the inputs and of
-// nothing else per tap (the taps of a thread's channels are read once).  Per element the arithmetic of the
-// kernel above.
+// Prompt portions: bfloat16 in, four neighbouring channels by SC_TILE consecutive rows a thread, 8-byte
+// accesses; every input row is read once for all the taps that want it (and the taps of a thread's channels once).  A
+// row's request is the same for all threads of a block, so the cases below are uniform branches.  Per element the
+// arithmetic of the kernel above.
+#define SC_TILE 8
 template <typename O, int K>
 __global__ void __launch_bounds__(256)
 short_conv_rows_kernel(O* __restrict__ out, const bf16_t* __restrict__ proj, int width, int first_col, int channels,
                        const bf16_t* __restrict__ taps, const bf16_t* __restrict__ bias, const float* __restrict__ state,
                        const int* __restrict__ state_slots, const int* __restrict__ token_seq,
-                       const int* __restrict__ query_start_loc, int activation) {
+                       const int* __restrict__ query_start_loc, int activation, int tokens) {
   const int c = 4 * (blockIdx.y * blockDim.x + threadIdx.x);
   if (c >= channels) return;
-  const int t = blockIdx.x;
-  const int seq = token_seq[t];
-  const int row0 = query_start_loc[seq];
-  const int index = t - row0;
-  constexpr int k = K;
-  const float* held = state + (size_t)state_slots[seq] * (k - 1) * channels + c;
-  float y[4] = {0.f, 0.f, 0.f, 0.f};
+  const int t0 = blockIdx.x * SC_TILE;
+  uint2 raw[SC_TILE + K - 1];  // rows t0 - (K - 1) .. t0 + SC_TILE - 1 of the projection
+#pragma unroll
+  for (int i = 0; i < SC_TILE + K - 1; ++i) {
+    const int row = min(max(t0 - (K - 1) + i, 0), tokens - 1);  // (a row outside is never looked at)
+    raw[i] = *reinterpret_cast<const uint2*>(proj + (size_t)row * width + first_col + c);
+  }
   // The 4 K taps of the thread's channels lie side by side: K loads of four.
-  float w[4 * K];
+  float w[4 * K], add[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int f = 0; f < K; ++f) {
-    const uint2 raw = *reinterpret_cast<const uint2*>(taps + (size_t)c * k + 4 * f);
-    w[4 * f] = __uint_as_float(raw.x << 16);
-    w[4 * f + 1] = __uint_as_float(raw.x & 0xffff0000u);
-    w[4 * f + 2] = __uint_as_float(raw.y << 16);
-    w[4 * f + 3] = __uint_as_float(raw.y & 0xffff0000u);
-  }
+    float four[4];
+    load_vec<bf16_t, 4>(taps + (size_t)c * K + 4 * f, four);
 #pragma unroll
-  for (int j = 0; j < K; ++j) {
-    const int back = index - (k - 1) + j;
-    float u[4];
-    if (back >= 0) {
-      const uint2 raw = *reinterpret_cast<const uint2*>(proj + (size_t)(row0 + back) * width + first_col + c);
-      u[0] = __uint_as_float(raw.x << 16);
-      u[1] = __uint_as_float(raw.x & 0xffff0000u);
-      u[2] = __uint_as_float(raw.y << 16);
-      u[3] = __uint_as_float(raw.y & 0xffff0000u);
-    } else {
-      const float4 raw = *reinterpret_cast<const float4*>(held + (size_t)(k - 1 + back) * channels);
-      u[0] = raw.x; u[1] = raw.y; u[2] = raw.z; u[3] = raw.w;
+    for (int e = 0; e < 4; ++e) w[4 * f + e] = four[e];
+  }
+  if (bias) load_vec<bf16_t, 4>(bias + c, add);
+#pragma unroll
+  for (int j = 0; j < SC_TILE; ++j) {
+    const int t = t0 + j;
+    if (t >= tokens) break;
+    const int seq = token_seq[t];
+    const int index = t - query_start_loc[seq];  // the token's place in its request's portion
+    float y[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int f = 0; f < K; ++f) {
+      const int back = index - (K - 1) + f;
+      float u[4];
+      if (back >= 0) {
+        const uint2 r = raw[j + f];
+        u[0] = __uint_as_float(r.x << 16);
+        u[1] = __uint_as_float(r.x & 0xffff0000u);
+        u[2] = __uint_as_float(r.y << 16);
+        u[3] = __uint_as_float(r.y & 0xffff0000u);
+      } else {
+        load_vec<float, 4>(state + ((size_t)state_slots[seq] * (K - 1) + K - 1 + back) * channels + c, u);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = fmaf(w[e * K + f], u[e], y[e]);
     }
 #pragma unroll
-    for (int e = 0; e < 4; ++e) y[e] = fmaf(w[e * K + j], u[e], y[e]);
-  }
-  if (bias) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) y[e] += to_float(bias[c + e]);
-  }
-#pragma unroll
-  for (int e = 0; e < 4; ++e)
-    if (activation == 1) y[e] = y[e] / (1.f + expf(-y[e]));
-  O* to = out + (size_t)t * channels + c;
-  if constexpr (sizeof(O) == 4) {
-    *reinterpret_cast<float4*>(to) = make_float4(y[0], y[1], y[2], y[3]);
-  } else {
-    uint2 packed;
-    packed.x = (uint32_t)from_float<bf16_t>(y[0]).bits | ((uint32_t)from_float<bf16_t>(y[1]).bits << 16);
-    packed.y = (uint32_t)from_float<bf16_t>(y[2]).bits | ((uint32_t)from_float<bf16_t>(y[3]).bits << 16);
-    *reinterpret_cast<uint2*>(to) = packed;
+    for (int e = 0; e < 4; ++e) {
+      if (bias) y[e] += add[e];
+      if (activation == 1) y[e] = y[e] / (1.f + expf(-y[e]));
+    }
+    store_vec<O, 4>(out + (size_t)t * channels + c, y);
   }
 }
 
@@ -161,15 +160,15 @@ extern "C" int ts_short_conv(void* out, int out_f32, const void* proj, int in_f3
   if (grid.y > 65535) return TS_ERR_SHAPE;
   if (dtype == TS_BF16 && !in_f32 && !single && tokens >= 32 && channels % 4 == 0 && width % 4 == 0 && first_col % 4 == 0 &&
       ((uintptr_t)proj | (uintptr_t)out | (uintptr_t)state | (uintptr_t)taps) % 16 == 0) {
-    const dim3 wide(tokens, (channels / 4 + 255) / 256);
+    const dim3 wide((tokens + SC_TILE - 1) / SC_TILE, (channels / 4 + 255) / 256);
 #define SC_ROWS(K)                                                                                                       \
   case K:                                                                                                                \
     if (out_f32)                                                                                                         \
       hipLaunchKernelGGL((short_conv_rows_kernel<float, K>), wide, block, 0, stream, (float*)out, (const bf16_t*)proj, width,       \
-                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation);  \
+                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation, tokens);  \
     else                                                                                                                 \
       hipLaunchKernelGGL((short_conv_rows_kernel<bf16_t, K>), wide, block, 0, stream, (bf16_t*)out, (const bf16_t*)proj, width,     \
-                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation);  \
+                         first_col, channels, (const bf16_t*)taps, (const bf16_t*)bias, state, state_slots, token_seq, query_start_loc, activation, tokens);  \
     break;
     switch (k) {
       SC_ROWS(1) SC_ROWS(2) SC_ROWS(3) SC_ROWS(4) SC_ROWS(5) SC_ROWS(6) SC_ROWS(7) SC_ROWS(8)

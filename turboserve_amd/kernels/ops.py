@@ -123,6 +123,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "ts_linear_state_finish": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_float, c_int, c_int, c_int,
                                    c_int, c_int, c_int, c_void_p],
         "ts_embed_positions": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_zero_state_rows": [c_void_p, c_int, c_void_p, c_int, c_void_p],
         "ts_copy_f32": [c_void_p, c_void_p, c_long, c_void_p],
         "ts_stream_offset": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
         "ts_moe_select": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
@@ -185,6 +186,16 @@ def load_module(module: str) -> ctypes.CDLL:
         fn.restype = c_int
     _LIBRARIES[module] = lib
     return lib
+
+
+def zero_state_rows(table: torch.Tensor, slots) -> None:
+    """Clear the rows ``slots`` (host integers, checked by the caller) of every tensor that ``table [n, 2]`` (int64 on the
+    device: address, bytes of a row) names, in one launch on the current stream."""
+    _gpu(table)
+    _need(table.dtype == torch.int64 and table.is_contiguous() and table.dim() == 2 and table.shape[1] == 2, "the table must be int64 [n, 2]")
+    host = (c_int * len(slots))(*slots)
+    _check(load_module("core").ts_zero_state_rows(_ptr(table), table.shape[0], host, len(slots),
+                                                  torch.cuda.current_stream(table.device).cuda_stream), "ts_zero_state_rows")
 
 
 def _ptr(t: torch.Tensor | None) -> int | None:
