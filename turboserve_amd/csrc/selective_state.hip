@@ -27,6 +27,7 @@
 #include "vec.hpp"
 
 #define SS_PIECE 128
+#define SS_STRETCH 32
 #define SS_PARTS 8  // lanes that share a column of the state in the walk
 
 typedef __bf16 ss_bf16x8 __attribute__((ext_vector_type(8)));
@@ -166,7 +167,8 @@ __device__ __forceinline__ void ss_cut(float v, uint32_t& top, uint32_t& mid, ui
   low = __float_as_uint(r1 - __uint_as_float(mid));
 }
 
-__device__ __forceinline__ uint32_t ss_pair(uint32_t lower, uint32_t upper) { return (lower >> 16) | (upper & 0xffff0000u); }
+// The upper halves of two words side by side.
+__device__ __forceinline__ uint32_t ss_pair(uint32_t lower, uint32_t upper) { return __builtin_amdgcn_perm(upper, lower, 0x07060302u); }
 
 __device__ __forceinline__ ss_f32x4 ss_mfma(ts_u32x4 a, ts_u32x4 b, ss_f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(ss_bf16x8, a), __builtin_bit_cast(ss_bf16x8, b), c, 0, 0, 0);
@@ -221,20 +223,31 @@ __device__ __forceinline__ void ss_load_rows(const bf16_t* u, size_t u_width, in
 
 __device__ __forceinline__ uint32_t ss_half(ts_u32x4 v, int e) { return e & 1 ? v[e / 2] & 0xffff0000u : v[e / 2] << 16; }  // as the bits of a float
 
+// Where mode 0 keeps token j of row r in LDS.  Rows are SS_STRETCH + 8 apart; the four chunks of eight tokens change
+// places by the row's group of eight, and groups of 32 rows are 16 words further apart: so the threads that turn tokens
+// and rows over, whose rows are eight apart, write to different banks.
+__device__ __forceinline__ int ss_place(int r, int j) {
+  return r * (SS_STRETCH + 8) + (r >> 5) * 32 + ((((j >> 3) ^ (r >> 3)) & 3) << 3) + (j & 7);
+}
+
+constexpr int ss_rows_size(int rows) { return rows * (SS_STRETCH + 8) + ((rows + 31) >> 5) * 32; }
+
 // Mode 0.  NK: stretches of 32 state rows; PT: stretches of 16 columns.  A wavefront owns every fourth stretch of 16
 // state rows and all columns: S_end^T (rows n, columns p) = sum over j of B^T (exact, LDS, tokens side by side) times
-// the weighted x (three planes, LDS).  The piece is taken in two halves of 64 tokens.
+// the weighted x (three planes, LDS).  The piece is taken in stretches of
+// SS_STRETCH tokens, so that four workgroups and more fit a compute unit.
 template <typename P, int NK, int PT>
 __global__ void __launch_bounds__(256)
 selective_piece_state_kernel(float* __restrict__ piece_state, float* __restrict__ piece_decay, const bf16_t* __restrict__ u,
                              const P* __restrict__ proj, int splits, size_t split_stride, int width, int dt_at,
                              const float* __restrict__ dt_bias, const float* __restrict__ a_log, const SsPiece* __restrict__ pieces,
                              int heads, int groups, int n, int p) {
-  constexpr int NP = 32 * NK, PP = 16 * PT, HALF = 64, ROW = HALF + 8;
+  constexpr int NP = 32 * NK, PP = 16 * PT;
   constexpr int TILES = (2 * NK + 3) / 4;  // stretches of 16 state rows a wavefront owns
   extern __shared__ __attribute__((aligned(16))) uint16_t ss_lds[];
-  uint16_t* bt = ss_lds;                // [NP][ROW]
-  uint16_t* xw = ss_lds + NP * ROW;     // [3][PP][ROW]
+  uint16_t* bt = ss_lds;                          // NP rows: B, tokens side by side
+  uint16_t* const xw[3] = {ss_lds + ss_rows_size(NP), ss_lds + ss_rows_size(NP) + ss_rows_size(PP),
+                           ss_lds + ss_rows_size(NP) + 2 * ss_rows_size(PP)};  // PP rows each: the weighted x in three planes
   __shared__ SsSteps steps;
   const int item = blockIdx.x, h = blockIdx.y, g = h / (heads / groups);
   const SsPiece piece = pieces[item];
@@ -249,58 +262,54 @@ selective_piece_state_kernel(float* __restrict__ piece_state, float* __restrict_
   for (int a = 0; a < TILES; ++a)
 #pragma unroll
     for (int b = 0; b < PT; ++b) acc[a][b] = ss_f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int half = 0; half < 2 && half * HALF < piece.count; ++half) {
-    __syncthreads();  // the steps are there; the half before has been read
-    const int j0 = half * HALF;
-    for (int i = tid; i < (HALF / 4) * (NP / 8); i += 256) {
-      const int q = i % (HALF / 4), d = (i / (HALF / 4)) * 8;
+  for (int j0 = 0; j0 < piece.count; j0 += SS_STRETCH) {
+    __syncthreads();  // the steps are there; the stretch before has been read
+    for (int i = tid; i < (SS_STRETCH / 4) * (NP / 8); i += 256) {
+      const int q = i / (NP / 8), d = (i % (NP / 8)) * 8;
       ts_u32x4 raw[4];
       ss_load_rows(u, u_width, piece.first, j0 + 4 * q, piece.count, b_at + d, d < n, raw);
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const ss_u32x2 four = {ss_pair(ss_half(raw[0], e), ss_half(raw[1], e)), ss_pair(ss_half(raw[2], e), ss_half(raw[3], e))};
-        *reinterpret_cast<ss_u32x2*>(&bt[(d + e) * ROW + 4 * q]) = four;
+        *reinterpret_cast<ss_u32x2*>(&bt[ss_place(d + e, 4 * q)]) = four;
       }
     }
     const float end_top = steps.top[SS_PIECE - 1], end_low = steps.low[SS_PIECE - 1];
-    for (int i = tid; i < (HALF / 4) * (PP / 8); i += 256) {
-      const int q = i % (HALF / 4), d = (i / (HALF / 4)) * 8;
-      ts_u32x4 raw[4];
-      ss_load_rows(u, u_width, piece.first, j0 + 4 * q, piece.count, x_at + d, c0 + d < p, raw);
-      float w[4];
+    for (int i = tid; i < (SS_STRETCH / 2) * (PP / 8); i += 256) {  // two tokens by eight columns a thread
+      const int q = i / (PP / 8), d = (i % (PP / 8)) * 8;
+      ts_u32x4 raw[2];
+      float w[2];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int j = j0 + 4 * q + e;
-        w[e] = steps.dt[j] * expf((end_top - steps.top[j]) + (end_low - steps.low[j]));
+      for (int k = 0; k < 2; ++k) {
+        const int j = j0 + 2 * q + k;
+        raw[k] = ts_u32x4{0u, 0u, 0u, 0u};
+        if (c0 + d < p && j < piece.count) raw[k] = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + j) * u_width + x_at + d);
+        w[k] = steps.dt[j] * expf((end_top - steps.top[j]) + (end_low - steps.low[j]));
       }
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        uint32_t top[4], mid[4], low[4];
+        uint32_t top[2], mid[2], low[2];
 #pragma unroll
-        for (int k = 0; k < 4; ++k) ss_cut(w[k] * __uint_as_float(ss_half(raw[k], e)), top[k], mid[k], low[k]);
-        *reinterpret_cast<ss_u32x2*>(&xw[(d + e) * ROW + 4 * q]) = ss_u32x2{ss_pair(top[0], top[1]), ss_pair(top[2], top[3])};
-        *reinterpret_cast<ss_u32x2*>(&xw[(PP + d + e) * ROW + 4 * q]) = ss_u32x2{ss_pair(mid[0], mid[1]), ss_pair(mid[2], mid[3])};
-        *reinterpret_cast<ss_u32x2*>(&xw[(2 * PP + d + e) * ROW + 4 * q]) = ss_u32x2{ss_pair(low[0], low[1]), ss_pair(low[2], low[3])};
+        for (int k = 0; k < 2; ++k) ss_cut(w[k] * __uint_as_float(ss_half(raw[k], e)), top[k], mid[k], low[k]);
+        const int at = ss_place(d + e, 2 * q);
+        *reinterpret_cast<uint32_t*>(&xw[0][at]) = ss_pair(top[0], top[1]);
+        *reinterpret_cast<uint32_t*>(&xw[1][at]) = ss_pair(mid[0], mid[1]);
+        *reinterpret_cast<uint32_t*>(&xw[2][at]) = ss_pair(low[0], low[1]);
       }
     }
     __syncthreads();
+    ts_u32x4 bf[TILES];
 #pragma unroll
-    for (int k = 0; k < HALF; k += 32) {
-      ts_u32x4 bf[TILES];
+    for (int a = 0; a < TILES; ++a)
+      bf[a] = *reinterpret_cast<const ts_u32x4*>(&bt[ss_place(16 * min(wave + 4 * a, 2 * NK - 1) + lo, 8 * quad)]);
 #pragma unroll
-      for (int a = 0; a < TILES; ++a) {
-        const int tile = min(wave + 4 * a, 2 * NK - 1);
-        bf[a] = *reinterpret_cast<const ts_u32x4*>(&bt[(16 * tile + lo) * ROW + k + 8 * quad]);
+    for (int plane = 2; plane >= 0; --plane)  // (the small planes first)
+#pragma unroll
+      for (int b = 0; b < PT; ++b) {
+        const ts_u32x4 xf = *reinterpret_cast<const ts_u32x4*>(&xw[plane][ss_place(16 * b + lo, 8 * quad)]);
+#pragma unroll
+        for (int a = 0; a < TILES; ++a) acc[a][b] = ss_mfma(bf[a], xf, acc[a][b]);
       }
-#pragma unroll
-      for (int plane = 2; plane >= 0; --plane)  // (the small planes first)
-#pragma unroll
-        for (int b = 0; b < PT; ++b) {
-          const ts_u32x4 xf = *reinterpret_cast<const ts_u32x4*>(&xw[(plane * PP + 16 * b + lo) * ROW + k + 8 * quad]);
-#pragma unroll
-          for (int a = 0; a < TILES; ++a) acc[a][b] = ss_mfma(bf[a], xf, acc[a][b]);
-        }
-    }
   }
 #pragma unroll
   for (int a = 0; a < TILES; ++a) {
@@ -358,18 +367,22 @@ selective_carry_kernel(float* __restrict__ state, const int* __restrict__ state_
 // other's two).  Everything is computed turned, y^T (rows p, columns i): the weights (C_i . B_j) exp(c_i - c_j) dt_j come
 // out of one product with token i on the lane and four tokens j in its registers, which is what the next product wants of
 // its second operand if the tokens j are counted in that order; they never leave the registers.
+// Of the tokens j before the stretch the factor is exp(c_i - c_r) times exp(c_r - c_j) dt_j, r the last token before
+// the stretch: the first is applied to a stretch's sums once, the second comes from a table that the workgroup makes once
+// (`before`: both exponents are at most zero, so nothing overflows however strong the decays are).
 template <typename P, int NK, int PT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, NK <= 4 ? 4 : 2)
 selective_piece_out_kernel(float* __restrict__ y, const float* __restrict__ piece_state, const bf16_t* __restrict__ u,
                            const P* __restrict__ proj, int splits, size_t split_stride, int width, int dt_at,
                            const float* __restrict__ dt_bias, const float* __restrict__ a_log, const float* __restrict__ skip,
                            const SsPiece* __restrict__ pieces, int heads, int groups, int n, int p) {
-  constexpr int NP = 32 * NK, PP = 16 * PT, SROW = NP + 8, XROW = SS_PIECE + 8;
+  constexpr int NP = 32 * NK, PP = 16 * PT, SROW = NP + 8, XROW = SS_PIECE + 4, HALF = SS_PIECE / 2;
   extern __shared__ __attribute__((aligned(16))) uint16_t ss_lds[];
-  uint16_t* planes = ss_lds;               // [3][PP][SROW]: the state before the piece
-  uint16_t* br = ss_lds;                   // then [SS_PIECE][SROW]: B
-  uint16_t* xt = ss_lds + SS_PIECE * SROW; // and [PP][XROW]: x, tokens side by side
+  uint16_t* planes = ss_lds;           // [2][PP][SROW]: the state before the piece, its two lower planes, then its upper one
+  uint16_t* br = ss_lds;               // then [HALF][SROW]: B of half the tokens at a time
+  uint16_t* xt = ss_lds + HALF * SROW; // and [PP][XROW]: x, tokens side by side
   __shared__ __attribute__((aligned(16))) SsSteps steps;
+  __shared__ __attribute__((aligned(16))) float before[SS_PIECE / 16][SS_PIECE];  // [stretch of i][j]
   const int item = blockIdx.x, h = blockIdx.y, g = h / (heads / groups);
   const SsPiece piece = pieces[item];
   const int tid = threadIdx.x, wave = tid / TS_WAVE, lane = tid % TS_WAVE;
@@ -378,137 +391,166 @@ selective_piece_out_kernel(float* __restrict__ y, const float* __restrict__ piec
   const size_t u_width = (size_t)heads * p + (size_t)2 * groups * n;
   const size_t b_at = (size_t)heads * p + (size_t)g * n, c_at = b_at + (size_t)groups * n, x_at = (size_t)h * p + c0;
   const int tiles[2] = {wave, 7 - wave};
-  // C of the wavefront's tokens: columns i, eight state rows a lane.
-  ts_u32x4 cf[2][NK];
-#pragma unroll
-  for (int a = 0; a < 2; ++a) {
-    const int i = 16 * tiles[a] + lo;
-#pragma unroll
-    for (int k = 0; k < NK; ++k) {
-      const int d = 32 * k + 8 * quad;
-      cf[a][k] = ts_u32x4{0u, 0u, 0u, 0u};
-      if (i < piece.count && d < n) cf[a][k] = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + i) * u_width + c_at + d);
-    }
-  }
   if (wave == 0) ss_steps(steps, proj, splits, split_stride, width, dt_at + h, dt_bias[h], expf(a_log[h]), piece);
-  const float* before = piece_state + (((size_t)item * heads + h) * p + c0) * n;
-  for (int i = tid; i < PP * (NP / 8); i += 256) {
-    const int c = i / (NP / 8), d = (i % (NP / 8)) * 8;
-    ts_u32x4 out[3] = {ts_u32x4{0u, 0u, 0u, 0u}, ts_u32x4{0u, 0u, 0u, 0u}, ts_u32x4{0u, 0u, 0u, 0u}};
-    if (c0 + c < p && d < n) {
-      const float4 v0 = *reinterpret_cast<const float4*>(before + (size_t)c * n + d);
-      const float4 v1 = *reinterpret_cast<const float4*>(before + (size_t)c * n + d + 4);
-      const float v[8] = {v0.x, v0.y, v0.z, v0.w, v1.x, v1.y, v1.z, v1.w};
-      uint32_t top[8], mid[8], low[8];
-#pragma unroll
-      for (int e = 0; e < 8; ++e) ss_cut(v[e], top[e], mid[e], low[e]);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        out[0][e] = ss_pair(top[2 * e], top[2 * e + 1]);
-        out[1][e] = ss_pair(mid[2 * e], mid[2 * e + 1]);
-        out[2][e] = ss_pair(low[2 * e], low[2 * e + 1]);
-      }
-    }
-#pragma unroll
-    for (int plane = 0; plane < 3; ++plane) *reinterpret_cast<ts_u32x4*>(&planes[(plane * PP + c) * SROW + d]) = out[plane];
-  }
-  __syncthreads();
+  const float* entering = piece_state + (((size_t)item * heads + h) * p + c0) * n;
+  ts_u32x4 cf[2][NK];  // C of the wavefront's tokens: columns i, eight state rows a lane
   ss_f32x4 acc[PT][2];
 #pragma unroll
   for (int b = 0; b < PT; ++b)
 #pragma unroll
     for (int a = 0; a < 2; ++a) acc[b][a] = ss_f32x4{0.f, 0.f, 0.f, 0.f};
+  constexpr int ITEMS = (PP * (NP / 8) + 255) / 256;
+  ts_u32x4 upper[ITEMS];  // the upper plane of what the thread has read of the state, while the lower ones are multiplied
 #pragma unroll
-  for (int plane = 2; plane >= 0; --plane)
+  for (int turn = 0; turn < 2; ++turn) {  // the two lower planes first, then the upper one in their place
+    if (turn > 0) __syncthreads();
 #pragma unroll
-    for (int k = 0; k < NK; ++k)
-#pragma unroll
-      for (int b = 0; b < PT; ++b) {
-        const ts_u32x4 sf = *reinterpret_cast<const ts_u32x4*>(&planes[(plane * PP + 16 * b + lo) * SROW + 32 * k + 8 * quad]);
-#pragma unroll
-        for (int a = 0; a < 2; ++a) acc[b][a] = ss_mfma(sf, cf[a][k], acc[b][a]);
+    for (int x = 0; x < ITEMS; ++x) {
+      const int i = tid + 256 * x;
+      if (i >= PP * (NP / 8)) continue;
+      const int c = i / (NP / 8), d = (i % (NP / 8)) * 8;
+      if (turn > 0) {
+        *reinterpret_cast<ts_u32x4*>(&planes[c * SROW + d]) = upper[x];
+        continue;
       }
-  float mine_top[2], mine_low[2];
+      float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (c0 + c < p && d < n) {
+        const float4 v0 = *reinterpret_cast<const float4*>(entering + (size_t)c * n + d);
+        const float4 v1 = *reinterpret_cast<const float4*>(entering + (size_t)c * n + d + 4);
+        v[0] = v0.x; v[1] = v0.y; v[2] = v0.z; v[3] = v0.w;
+        v[4] = v1.x; v[5] = v1.y; v[6] = v1.z; v[7] = v1.w;
+      }
+      ts_u32x4 middle, lower;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        uint32_t top[2], mid[2], low[2];
+        ss_cut(v[2 * e], top[0], mid[0], low[0]);
+        ss_cut(v[2 * e + 1], top[1], mid[1], low[1]);
+        upper[x][e] = ss_pair(top[0], top[1]);
+        middle[e] = ss_pair(mid[0], mid[1]);
+        lower[e] = ss_pair(low[0], low[1]);
+      }
+      *reinterpret_cast<ts_u32x4*>(&planes[c * SROW + d]) = middle;
+      *reinterpret_cast<ts_u32x4*>(&planes[(PP + c) * SROW + d]) = lower;
+    }
+    if (turn == 0) {
+#pragma unroll
+      for (int a = 0; a < 2; ++a) {
+        const int i = 16 * tiles[a] + lo;
+#pragma unroll
+        for (int k = 0; k < NK; ++k) {
+          const int d = 32 * k + 8 * quad;
+          cf[a][k] = ts_u32x4{0u, 0u, 0u, 0u};
+          if (i < piece.count && d < n) cf[a][k] = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + i) * u_width + c_at + d);
+        }
+      }
+    }
+    __syncthreads();
+    if (turn == 0) {
+#pragma unroll 1
+      for (int i = tid; i < SS_PIECE / 16 * SS_PIECE; i += 256) {
+        const int tile = i / SS_PIECE, j = i % SS_PIECE, r = 16 * tile - 1;
+        if (j <= r) before[tile][j] = steps.dt[j] * __expf((steps.top[r] - steps.top[j]) + (steps.low[r] - steps.low[j]));
+      }
+    }
+#pragma unroll
+    for (int plane = 1 - turn; plane >= 0; --plane)
+#pragma unroll
+      for (int k = 0; k < NK; ++k)
+#pragma unroll
+        for (int b = 0; b < PT; ++b) {
+          const ts_u32x4 sf = *reinterpret_cast<const ts_u32x4*>(&planes[(plane * PP + 16 * b + lo) * SROW + 32 * k + 8 * quad]);
+#pragma unroll
+          for (int a = 0; a < 2; ++a) acc[b][a] = ss_mfma(sf, cf[a][k], acc[b][a]);
+        }
+  }
 #pragma unroll
   for (int a = 0; a < 2; ++a) {
-    const int i = 16 * tiles[a] + lo;
-    mine_top[a] = steps.top[i];
-    mine_low[a] = steps.low[i];
-    const float by = expf(mine_top[a] + mine_low[a]);
+    const float by = tiles[a] > 0 ? expf(steps.top[16 * tiles[a] - 1] + steps.low[16 * tiles[a] - 1]) : 1.f;
 #pragma unroll
     for (int b = 0; b < PT; ++b) acc[b][a] *= by;
   }
-  __syncthreads();  // the planes have been read: their place takes B and x
-  for (int i = tid; i < SS_PIECE * (NP / 8); i += 256) {
-    const int j = i / (NP / 8), d = (i % (NP / 8)) * 8;
-    ts_u32x4 raw = {0u, 0u, 0u, 0u};
-    if (j < piece.count && d < n) raw = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + j) * u_width + b_at + d);
-    *reinterpret_cast<ts_u32x4*>(&br[j * SROW + d]) = raw;
-  }
-  for (int i = tid; i < (SS_PIECE / 4) * (PP / 8); i += 256) {
-    const int q = i % (SS_PIECE / 4), d = (i / (SS_PIECE / 4)) * 8;
-    ts_u32x4 raw[4];
-    ss_load_rows(u, u_width, piece.first, 4 * q, piece.count, x_at + d, c0 + d < p, raw);
-#pragma unroll
-    for (int e = 0; e < 8; ++e)
-      *reinterpret_cast<ss_u32x2*>(&xt[(d + e) * XROW + 4 * q]) =
-          ss_u32x2{ss_pair(ss_half(raw[0], e), ss_half(raw[1], e)), ss_pair(ss_half(raw[2], e), ss_half(raw[3], e))};
-  }
-  __syncthreads();
-  for (int jb = 0; 32 * jb < piece.count; ++jb) {
-    if (2 * jb > tiles[1] || 16 * tiles[0] >= piece.count) break;  // (the later stretch sees no further token; no token is the wavefront's)
-    const bool early = 2 * jb <= tiles[0];
-    ss_f32x4 s[2][2];  // [stretch of 16 tokens j][stretch of tokens i]
-#pragma unroll
-    for (int t = 0; t < 2; ++t)
-#pragma unroll
-      for (int a = 0; a < 2; ++a) s[t][a] = ss_f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int k = 0; k < NK; ++k)
-#pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        const ts_u32x4 bf = *reinterpret_cast<const ts_u32x4*>(&br[(32 * jb + 16 * t + lo) * SROW + 32 * k + 8 * quad]);
-        if (early) s[t][0] = ss_mfma(bf, cf[0][k], s[t][0]);
-        s[t][1] = ss_mfma(bf, cf[1][k], s[t][1]);
-      }
-    ts_u32x4 xf[PT];
-#pragma unroll
-    for (int b = 0; b < PT; ++b) {
-      const uint16_t* row = &xt[(16 * b + lo) * XROW + 32 * jb + 4 * quad];
-      const ss_u32x2 first = *reinterpret_cast<const ss_u32x2*>(row), second = *reinterpret_cast<const ss_u32x2*>(row + 16);
-      xf[b] = ts_u32x4{first[0], first[1], second[0], second[1]};
+  for (int half = 0; half * HALF < piece.count; ++half) {
+    __syncthreads();  // the planes, or B of the first half, have been read: their place takes what follows
+#pragma unroll 2
+    for (int i = tid; i < HALF * (NP / 8); i += 256) {
+      const int j = i / (NP / 8), d = (i % (NP / 8)) * 8;
+      ts_u32x4 raw = {0u, 0u, 0u, 0u};
+      if (half * HALF + j < piece.count && d < n)
+        raw = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + half * HALF + j) * u_width + b_at + d);
+      *reinterpret_cast<ts_u32x4*>(&br[j * SROW + d]) = raw;
     }
+#pragma unroll 1
+    for (int i = tid; half == 0 && i < (SS_PIECE / 2) * (PP / 8); i += 256) {  // two tokens by eight columns a thread
+      const int q = i / (PP / 8), d = (i % (PP / 8)) * 8;
+      ts_u32x4 raw[2];
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        raw[k] = ts_u32x4{0u, 0u, 0u, 0u};
+        if (c0 + d < p && 2 * q + k < piece.count)
+          raw[k] = *reinterpret_cast<const ts_u32x4*>(u + (size_t)(piece.first + 2 * q + k) * u_width + x_at + d);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        *reinterpret_cast<uint32_t*>(&xt[(d + e) * XROW + 2 * q]) = ss_pair(ss_half(raw[0], e), ss_half(raw[1], e));
+    }
+    __syncthreads();
 #pragma unroll
     for (int a = 0; a < 2; ++a) {
-      if (a == 0 && !early) continue;
-      const int i = 16 * tiles[a] + lo;
-      uint32_t top[8], mid[8], low[8];
+      const int tile = tiles[a];
+      if (16 * tile >= piece.count) continue;
+#pragma unroll 1
+      for (int jb = 2 * half; jb < 2 * half + 2 && 2 * jb <= tile; ++jb) {
+        ss_f32x4 s[2] = {ss_f32x4{0.f, 0.f, 0.f, 0.f}, ss_f32x4{0.f, 0.f, 0.f, 0.f}};  // by stretch of 16 tokens j
 #pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        const int j0 = 32 * jb + 16 * t + 4 * quad;
-        const float4 jt = *reinterpret_cast<const float4*>(&steps.top[j0]);
-        const float4 jl = *reinterpret_cast<const float4*>(&steps.low[j0]);
-        const float4 jd = *reinterpret_cast<const float4*>(&steps.dt[j0]);
-        const float tops[4] = {jt.x, jt.y, jt.z, jt.w}, lows[4] = {jl.x, jl.y, jl.z, jl.w}, dts[4] = {jd.x, jd.y, jd.z, jd.w};
+        for (int k = 0; k < NK; ++k)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          // (A later token's decay is never formed: its exponent would be positive.)
-          const float gone = j0 + r <= i ? (mine_top[a] - tops[r]) + (mine_low[a] - lows[r]) : 0.f;
-          const float w = j0 + r <= i ? s[t][a][r] * dts[r] * __expf(gone) : 0.f;
-          ss_cut(w, top[4 * t + r], mid[4 * t + r], low[4 * t + r]);
+          for (int t = 0; t < 2; ++t)
+            s[t] = ss_mfma(*reinterpret_cast<const ts_u32x4*>(&br[(32 * (jb - 2 * half) + 16 * t + lo) * SROW + 32 * k + 8 * quad]), cf[a][k], s[t]);
+        const int j0 = 32 * jb + 4 * quad;
+        if (2 * jb + 1 < tile) {
+#pragma unroll
+          for (int t = 0; t < 2; ++t) s[t] *= *reinterpret_cast<const ss_f32x4*>(&before[tile][j0 + 16 * t]);
+        } else {
+          // The stretch's own tokens (and, of an odd one, the sixteen before it): from here on the sums are y's own.
+          const int i = 16 * tile + lo;
+          const float mine_top = steps.top[i], mine_low = steps.low[i];
+          const float by = tile > 0 ? expf((mine_top - steps.top[16 * tile - 1]) + (mine_low - steps.low[16 * tile - 1])) : expf(mine_top + mine_low);
+#pragma unroll
+          for (int b = 0; b < PT; ++b) acc[b][a] *= by;
+#pragma unroll
+          for (int t = 0; t < 2; ++t) {
+            const ss_f32x4 tops = *reinterpret_cast<const ss_f32x4*>(&steps.top[j0 + 16 * t]);
+            const ss_f32x4 lows = *reinterpret_cast<const ss_f32x4*>(&steps.low[j0 + 16 * t]);
+            const ss_f32x4 dts = *reinterpret_cast<const ss_f32x4*>(&steps.dt[j0 + 16 * t]);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              // (A later token's decay is never formed: its exponent would be positive.)
+              const bool seen = j0 + 16 * t + r <= i;
+              const float gone = seen ? (mine_top - tops[r]) + (mine_low - lows[r]) : 0.f;
+              s[t][r] = seen ? s[t][r] * dts[r] * __expf(gone) : 0.f;
+            }
+          }
+        }
+        ts_u32x4 wf[3];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          uint32_t top[2], mid[2], low[2];
+#pragma unroll
+          for (int k = 0; k < 2; ++k) ss_cut(s[e / 2][2 * (e % 2) + k], top[k], mid[k], low[k]);
+          wf[0][e] = ss_pair(top[0], top[1]);
+          wf[1][e] = ss_pair(mid[0], mid[1]);
+          wf[2][e] = ss_pair(low[0], low[1]);
+        }
+#pragma unroll
+        for (int b = 0; b < PT; ++b) {
+          const uint16_t* row = &xt[(16 * b + lo) * XROW + j0];
+          const ss_u32x2 first = *reinterpret_cast<const ss_u32x2*>(row), second = *reinterpret_cast<const ss_u32x2*>(row + 16);
+          const ts_u32x4 xf = {first[0], first[1], second[0], second[1]};
+#pragma unroll
+          for (int plane = 2; plane >= 0; --plane) acc[b][a] = ss_mfma(xf, wf[plane], acc[b][a]);
         }
       }
-      ts_u32x4 wf[3];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        wf[0][e] = ss_pair(top[2 * e], top[2 * e + 1]);
-        wf[1][e] = ss_pair(mid[2 * e], mid[2 * e + 1]);
-        wf[2][e] = ss_pair(low[2 * e], low[2 * e + 1]);
-      }
-#pragma unroll
-      for (int plane = 2; plane >= 0; --plane)
-#pragma unroll
-        for (int b = 0; b < PT; ++b) acc[b][a] = ss_mfma(xf[b], wf[plane], acc[b][a]);
     }
   }
   const float d_skip = skip[h];
@@ -635,8 +677,8 @@ extern "C" int ts_selective_pieces(float* y, float* piece_state, float* piece_de
 #define SS_PIECES(P, NK, PT)                                                                                                         \
   do {                                                                                                                               \
     const dim3 grid(num_pieces, heads, (p + 16 * PT - 1) / (16 * PT));                                                               \
-    constexpr int state_lds = (32 * NK + 3 * 16 * PT) * 72 * 2;                                                                      \
-    constexpr int planes = 3 * 16 * PT * (32 * NK + 8) * 2, rows = (SS_PIECE * (32 * NK + 8) + 16 * PT * (SS_PIECE + 8)) * 2;        \
+    constexpr int state_lds = (ss_rows_size(32 * NK) + 3 * ss_rows_size(16 * PT)) * 2;                                                                      \
+    constexpr int planes = 2 * 16 * PT * (32 * NK + 8) * 2, rows = (SS_PIECE / 2 * (32 * NK + 8) + 16 * PT * (SS_PIECE + 4)) * 2;    \
     constexpr int out_lds = planes > rows ? planes : rows;                                                                           \
     if (mode == 0) {                                                                                                                 \
       static const bool ready = hipFuncSetAttribute((const void*)selective_piece_state_kernel<P, NK, PT>,                            \

@@ -68,7 +68,7 @@ short_conv_kernel(O* __restrict__ out, const P* __restrict__ proj, int splits, s
 // Prompt portions: bfloat16 in, four neighbouring channels by SC_TILE consecutive rows a thread, 8-byte
 // accesses; every input row is read once for all the taps that want it (and the taps of a thread's channels once).  A
 // row's request is the same for all threads of a block, so the cases below are uniform branches.  Per element the
-// arithmetic of the kernel above.
+// sums of the kernel above.
 #define SC_TILE 8
 template <typename O, int K>
 __global__ void __launch_bounds__(256)
@@ -121,7 +121,8 @@ short_conv_rows_kernel(O* __restrict__ out, const bf16_t* __restrict__ proj, int
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       if (bias) y[e] += add[e];
-      if (activation == 1) y[e] = y[e] / (1.f + expf(-y[e]));
+      // (The hardware's exponential and reciprocal: an ulp or two of 32-bit.)
+      if (activation == 1) y[e] *= __builtin_amdgcn_rcpf(1.f + __expf(-y[e]));
     }
     store_vec<O, 4>(out + (size_t)t * channels + c, y);
   }

@@ -4,6 +4,9 @@
 
 #include "common.hpp"
 
+typedef __bf16 vec_bf16x2 __attribute__((ext_vector_type(2)));
+typedef float vec_f32x2 __attribute__((ext_vector_type(2)));
+
 template <typename P, int VEC>
 __device__ __forceinline__ void load_vec(const P* p, float (&v)[VEC]) {
   if constexpr (VEC == 4 && sizeof(P) == 4) {
@@ -26,10 +29,10 @@ __device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
   if constexpr (VEC == 4 && sizeof(T) == 4) {
     *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
   } else if constexpr (VEC == 4) {
-    uint2 packed;
-    packed.x = (uint32_t)from_float<bf16_t>(v[0]).bits | ((uint32_t)from_float<bf16_t>(v[1]).bits << 16);
-    packed.y = (uint32_t)from_float<bf16_t>(v[2]).bits | ((uint32_t)from_float<bf16_t>(v[3]).bits << 16);
-    *reinterpret_cast<uint2*>(p) = packed;
+    // (Round to nearest even, two elements an instruction.)
+    const vec_bf16x2 low = __builtin_convertvector(vec_f32x2{v[0], v[1]}, vec_bf16x2);
+    const vec_bf16x2 high = __builtin_convertvector(vec_f32x2{v[2], v[3]}, vec_bf16x2);
+    *reinterpret_cast<uint2*>(p) = make_uint2(__builtin_bit_cast(uint32_t, low), __builtin_bit_cast(uint32_t, high));
   } else {
 #pragma unroll
     for (int e = 0; e < VEC; ++e) p[e] = from_float<T>(v[e]);
