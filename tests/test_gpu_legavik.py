@@ -112,7 +112,7 @@ def test_the_norm_without_statistics_carries_the_residual_sum(ops, dtype, hidden
 
 def test_the_cap_on_the_logits(ops):
     x = torch.linspace(-90, 90, 1001).reshape(7, 143).contiguous()
-    near(ops.tanh_cap(x.clone().to(DEV), 22.0), 22.0 * torch.tanh(x / 22.0), torch.float32)
+    near(ops.scale_cap(x.clone().to(DEV), cap=22.0), 22.0 * torch.tanh(x / 22.0), torch.float32)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])

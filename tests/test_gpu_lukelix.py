@@ -261,7 +261,7 @@ def test_the_selective_state_whole_in_pieces_and_walked(ops, dtype, heads, group
     ds = [(2 * torch.randn(m, at + heads + 2, generator=g)).to(dtype) for m in lengths]
     want = [plain_selective(u.double(), d[:, at:at + heads].double(), t, heads, groups, n, p).float() for u, d in zip(us, ds)]
     on = {k: v.to(DEV) for k, v in t.items()}
-    pieces = ops.selective_pieces_supported(dtype, n, p)
+    pieces = ops.decaying_pieces_supported(dtype, n, p)
     assert pieces == (dtype == torch.bfloat16 and (n, p) in ((24, 16), (64, 64), (128, 48), (136, 8), (256, 72), (48, 40)))
     for sizes in ([1000], [128, 60, 2, 40, 1], [257, 3]):
         state = torch.full((6, heads, p, n), float("nan"), device=DEV)
@@ -280,7 +280,7 @@ def test_the_selective_state_whole_in_pieces_and_walked(ops, dtype, heads, group
                 starts.append(starts[-1] + counts[i])
             plan = None
             if pieces and long and turn % 3:
-                cut, carries = ops.linear_state_pieces([counts[i] for i in live[:long]], ops.selective_piece)
+                cut, carries = ops.linear_state_pieces([counts[i] for i in live[:long]], ops.decaying_piece)
                 plan = (ops.device_ints(cut), ops.device_ints(carries), len(cut), len(carries))
             y = ops.selective_state(u, given, at, on["dt_bias"], on["a_log"], on["skip"], state, ints([slots[i] for i in live]), ints(starts),
                                     num_seqs=len(live), heads=heads, groups=groups, state_dim=n, value_dim=p, dtype=dtype, plan=plan).cpu()

@@ -79,3 +79,8 @@ def _ensure_builtin() -> None:
         from turboserve_amd.models.lukelix import lukelix_plan
 
         register_architecture("Lukelix", LukelixConfig.from_dict, lukelix_plan)
+    if "Ninenex" not in ARCHITECTURES:
+        from turboserve_amd.config.ninenex_config import NinenexConfig
+        from turboserve_amd.models.ninenex import ninenex_plan
+
+        register_architecture("Ninenex", NinenexConfig.from_dict, ninenex_plan)

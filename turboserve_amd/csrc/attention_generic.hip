@@ -36,7 +36,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
                                int heads, int kv_heads, int dim, int vdim, int block_size, float scale,
                                float softcap, int window, const float* __restrict__ slopes, int chunk, float sinks,
                                const float* __restrict__ sink_scores, const float* __restrict__ distance_bias,
-                               int bias_len, int keep_first) {
+                               int bias_len, int keep_first, long out_stride, float out_scale) {
   __shared__ float qs[ATTN_MAX_DIM];
   __shared__ float ps[ATTN_TILE];
   __shared__ long long rows[ATTN_TILE];  // per key of the tile: offset of its value column
@@ -113,8 +113,8 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
   }
   }
 
-  T* orow = out + ((size_t)t * heads + h) * vdim;
-  const float inv = 1.f / l_run;
+  T* orow = out + (size_t)t * out_stride + (size_t)h * vdim;
+  const float inv = out_scale / l_run;
 #pragma unroll
   for (int c = 0; c < CHUNKS; ++c) {
     const int d = lane + c * ATTN_TILE;
@@ -122,7 +122,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
   }
 }
 
-// out [T, Hq, Dv] contiguous; q rows are q_stride elements apart (the fused projection output).
+// out: rows of [Hq, Dv], out_stride elements apart, times out_scale; q rows are q_stride elements apart (the fused projection output).
 // slopes [Hq] (32-bit) or null: the score of key j for the query at position p gets
 // slopes[h] * (j - p) added.  v_pages null: the values are the keys' first vdim elements.
 // sink_scores [Hq] (32-bit) or null; distance_bias [Hq, bias_len] (32-bit) or null.
@@ -133,10 +133,12 @@ extern "C" int ts_paged_attention_generic(void* out, const void* q, long q_strid
                                           int heads, int kv_heads, int dim, int vdim, int block_size,
                                           float scale, float softcap, int window, const float* slopes, int chunk,
                                           float sinks, const float* sink_scores, const float* distance_bias,
-                                          int bias_len, int keep_first, int dtype, hipStream_t stream) {
+                                          int bias_len, int keep_first, int dtype, long out_stride, float out_scale,
+                                          hipStream_t stream) {
   if (tokens == 0) return TS_OK;
   if (keep_first < 0 || (keep_first > 0 && chunk > 0)) return TS_ERR_ARG;
   if (!out || !q || !k_pages || !block_table || !token_seq || !positions) return TS_ERR_ARG;
+  if (out_stride < (long)heads * vdim) return TS_ERR_ARG;
   if (chunk < 0 || !(sinks >= 0.f) || (!v_pages && vdim > dim)) return TS_ERR_ARG;
   if ((sink_scores && !(sinks > 0.f)) || (distance_bias && bias_len < 1)) return TS_ERR_ARG;
   if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || heads > 65535) return TS_ERR_SHAPE;
@@ -144,9 +146,9 @@ extern "C" int ts_paged_attention_generic(void* out, const void* q, long q_strid
     return TS_ERR_SHAPE;
   dim3 grid(tokens, heads), block(ATTN_TILE);
   if (dtype == TS_F32)
-    hipLaunchKernelGGL(paged_attention_generic_kernel<float>, grid, block, 0, stream, (float*)out, (const float*)q, q_stride, (const float*)k_pages, (const float*)v_pages, block_table, table_width, token_seq, positions, heads, kv_heads, dim, vdim, block_size, scale, softcap, window, slopes, chunk, sinks, sink_scores, distance_bias, bias_len, keep_first);
+    hipLaunchKernelGGL(paged_attention_generic_kernel<float>, grid, block, 0, stream, (float*)out, (const float*)q, q_stride, (const float*)k_pages, (const float*)v_pages, block_table, table_width, token_seq, positions, heads, kv_heads, dim, vdim, block_size, scale, softcap, window, slopes, chunk, sinks, sink_scores, distance_bias, bias_len, keep_first, out_stride, out_scale);
   else if (dtype == TS_BF16)
-    hipLaunchKernelGGL(paged_attention_generic_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)out, (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_table, table_width, token_seq, positions, heads, kv_heads, dim, vdim, block_size, scale, softcap, window, slopes, chunk, sinks, sink_scores, distance_bias, bias_len, keep_first);
+    hipLaunchKernelGGL(paged_attention_generic_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)out, (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_table, table_width, token_seq, positions, heads, kv_heads, dim, vdim, block_size, scale, softcap, window, slopes, chunk, sinks, sink_scores, distance_bias, bias_len, keep_first, out_stride, out_scale);
   else
     return TS_ERR_DTYPE;
   return ts_launch_status();

@@ -38,6 +38,12 @@ struct FaRule {
   int keep;  // the keys 0 .. keep - 1 are seen also below the window's lower bound
 };
 
+// Where a token's heads go: rows `stride` elements apart (a stretch of columns of a wider buffer), times a scale.
+struct FaOut {
+  long stride;
+  float scale;
+};
+
 // Sum and maximum over the 16 lanes that hold one row of an accumulator tile (a row of lanes for
 // the data-parallel moves): every lane returns its row's result.
 __device__ __forceinline__ float row16_sum(float v) {
@@ -72,7 +78,7 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
                        const int* __restrict__ query_start_loc, const int* __restrict__ context_lens,
                        const int* __restrict__ tiles, int first_seq, int heads, int kv_heads, int dk, int dv,
                        int block_size, const float* __restrict__ slopes, FaRule rule, int splits,
-                       const float* __restrict__ sink_scores, const float* __restrict__ distance_bias, int bias_len) {
+                       const float* __restrict__ sink_scores, const float* __restrict__ distance_bias, int bias_len, FaOut placed) {
   extern __shared__ __attribute__((aligned(16))) uint16_t fa_lds[];
   constexpr int K_ROW = KD * 32 + FA_PAD;       // elements of a staged key row
   constexpr int V_ROW = FA_KEYS + FA_PAD;       // elements of a staged value column (64 keys)
@@ -362,8 +368,8 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
     const int r = wave * 16 + 4 * group + i;
     if (r >= tile_rows) continue;
     if (splits == 1) {
-      const float inv = l_run[i] > 0.f ? 1.f / l_run[i] : 0.f;
-      uint16_t* dst = out + ((size_t)row_token(r) * heads + row_head(r)) * dv;
+      const float inv = l_run[i] > 0.f ? placed.scale / l_run[i] : 0.f;
+      uint16_t* dst = out + (size_t)row_token(r) * placed.stride + (size_t)row_head(r) * dv;
 #pragma unroll
       for (int vt = 0; vt < VD; ++vt)
         if (16 * vt + r16 < dv) dst[16 * vt + r16] = from_float<bf16_t>(o[vt][i] * inv).bits;
@@ -389,7 +395,7 @@ __global__ void __launch_bounds__(128)
 attention_tiles_combine_kernel(uint16_t* __restrict__ out, const float* __restrict__ partial_o,
                                const float* __restrict__ partial_ml, const int* __restrict__ query_start_loc,
                                int first_seq, int heads, int dv, int splits, float sinks,
-                               const float* __restrict__ sink_scores) {
+                               const float* __restrict__ sink_scores, FaOut placed) {
   __shared__ float weight[FA_MAX_SPLITS];
   __shared__ float scratch[16];
   const int item = blockIdx.x, h = blockIdx.y;
@@ -402,7 +408,7 @@ attention_tiles_combine_kernel(uint16_t* __restrict__ out, const float* __restri
   const float w = ms == -INFINITY ? 0.f : expf(ms - m);
   if (sp < splits) weight[sp] = w;
   const float l = block_sum(ls * w, scratch) + (sinks > 0.f ? sinks * expf(sink_at - m) : 0.f);  // (its barriers publish the weights)
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = l > 0.f ? placed.scale / l : 0.f;
   const int row = query_start_loc[first_seq + item];
   for (int d = threadIdx.x; d < dv; d += blockDim.x) {
     float acc = 0.f;
@@ -414,7 +420,7 @@ attention_tiles_combine_kernel(uint16_t* __restrict__ out, const float* __restri
       for (int j = 0; j < 8; ++j)
         if (first + j < splits) acc = fmaf(v[j], weight[first + j], acc);
     }
-    out[((size_t)row * heads + h) * dv + d] = from_float<bf16_t>(acc * inv).bits;
+    out[(size_t)row * placed.stride + (size_t)h * dv + d] = from_float<bf16_t>(acc * inv).bits;
   }
 }
 
@@ -424,7 +430,7 @@ static int tiles_launch(bool single, bool values_in_keys, dim3 grid, hipStream_t
                         const uint16_t* v_pages, const int* block_table, int table_width, const int* query_start_loc,
                         const int* context_lens, const int* tiles, int first_seq, int heads, int kv_heads, int dk, int dv,
                         int block_size, const float* slopes, FaRule rule, int splits, const float* sink_scores,
-                        const float* distance_bias, int bias_len) {
+                        const float* distance_bias, int bias_len, FaOut placed) {
   constexpr size_t lds = (size_t)(FA_KEYS * (KD * 32 + FA_PAD) + VD * 16 * (FA_KEYS + FA_PAD) + 4 * 16 * (FA_KEYS + FA_PAD)) * sizeof(uint16_t);
   static_assert(lds <= 160 * 1024, "the staged tiles must fit in LDS");
 #define FA_GO(SINGLE, INKEYS)                                                                                          \
@@ -439,7 +445,7 @@ static int tiles_launch(bool single, bool values_in_keys, dim3 grid, hipStream_t
     hipLaunchKernelGGL((attention_tiles_kernel<KD, VD, SINGLE, INKEYS>), grid, dim3(FA_THREADS), lds, stream, out,     \
                        partial_o, partial_ml, q, q_stride, k_pages, v_pages, block_table, table_width, query_start_loc, \
                        context_lens, tiles, first_seq, heads, kv_heads, dk, dv, block_size, slopes, rule, splits,      \
-                       sink_scores, distance_bias, bias_len);                                                          \
+                       sink_scores, distance_bias, bias_len, placed);                                                  \
   } while (0)
   if (single && values_in_keys) FA_GO(true, true);
   else if (single) FA_GO(true, false);
@@ -451,7 +457,8 @@ static int tiles_launch(bool single, bool values_in_keys, dim3 grid, hipStream_t
 
 // mode 0: prompt portions, `items` tiles (pairs: request, first row), each for every head;
 // mode 1: `items` requests of one token each from `first_seq` on, their keys shared out over `splits`.
-// out [T, heads, Dv] bfloat16.  v_pages null: the values are the keys' first Dv elements.
+// out: rows of [heads, Dv] bfloat16, `out_stride` elements apart; what is written is multiplied by out_scale (single
+// tokens whose keys are shared out: by the combining kernel).  v_pages null: the values are the keys' first Dv elements.
 // sink_scores [heads] (32-bit) or null: the score of the sinks, 0 without; distance_bias [heads, bias_len]
 // (32-bit) or null: the score of a key at distance n gets distance_bias[h][min(n, bias_len - 1)] added.
 extern "C" int ts_attention_tiles(void* out, void* partial_o, void* partial_ml, const void* q, long q_stride,
@@ -460,13 +467,13 @@ extern "C" int ts_attention_tiles(void* out, void* partial_o, void* partial_ml, 
                                   int first_seq, int heads, int kv_heads, int dk, int dv, int block_size, float scale,
                                   float softcap, int window, int chunk, float sinks, const float* slopes, int mode,
                                   int splits, const float* sink_scores, const float* distance_bias, int bias_len,
-                                  int keep_first, hipStream_t stream) {
+                                  int keep_first, long out_stride, float out_scale, hipStream_t stream) {
   if (items == 0) return TS_OK;
   if (keep_first < 0 || (keep_first > 0 && chunk > 0)) return TS_ERR_ARG;
   if (!out || !q || !k_pages || !block_table || !query_start_loc || !context_lens) return TS_ERR_ARG;
   if (mode == 0 && (!tiles || splits != 1)) return TS_ERR_ARG;
   if (mode == 1 && splits > 1 && (!partial_o || !partial_ml)) return TS_ERR_ARG;
-  if (mode < 0 || mode > 1 || splits < 1 || splits > FA_MAX_SPLITS) return TS_ERR_ARG;
+  if (mode < 0 || mode > 1 || splits < 1 || splits > FA_MAX_SPLITS || out_stride < (long)heads * dv) return TS_ERR_ARG;
   if ((sink_scores && !(sinks > 0.f)) || (distance_bias && (bias_len < 1 || !v_pages))) return TS_ERR_ARG;
   if (heads < 1 || kv_heads < 1 || heads % kv_heads != 0 || heads > 65535) return TS_ERR_SHAPE;
   if (dk < 8 || dk > 448 || dk % 8 != 0 || dv < 8 || dv > 384 || dv % 8 != 0 || block_size < 8 || block_size % 8 != 0)
@@ -485,7 +492,7 @@ extern "C" int ts_attention_tiles(void* out, void* partial_o, void* partial_ml, 
   return tiles_launch<KD, VD>(single, in_keys, grid, stream, (uint16_t*)out, (float*)partial_o, (float*)partial_ml,     \
                               (const uint16_t*)q, q_stride, (const uint16_t*)k_pages, (const uint16_t*)v_pages,         \
                               block_table, table_width, query_start_loc, context_lens, tiles, first_seq, heads, kv_heads, \
-                              dk, dv, block_size, slopes, rule, splits, sink_scores, distance_bias, bias_len)
+                              dk, dv, block_size, slopes, rule, splits, sink_scores, distance_bias, bias_len, FaOut{out_stride, out_scale})
   if (kd <= 2 && vd <= 4) FA_SIZE(2, 4);
   if (kd <= 4 && vd <= 8) FA_SIZE(4, 8);
   if (kd <= 4 && vd <= 16) FA_SIZE(4, 16);
@@ -500,11 +507,14 @@ extern "C" int ts_attention_tiles(void* out, void* partial_o, void* partial_ml, 
 
 extern "C" int ts_attention_tiles_combine(void* out, const void* partial_o, const void* partial_ml,
                                           const int* query_start_loc, int items, int first_seq, int heads, int dv,
-                                          int splits, float sinks, const float* sink_scores, hipStream_t stream) {
+                                          int splits, float sinks, const float* sink_scores, long out_stride, float out_scale,
+                                          hipStream_t stream) {
   if (items == 0) return TS_OK;
-  if (!out || !partial_o || !partial_ml || !query_start_loc || splits < 1 || splits > FA_MAX_SPLITS || heads < 1 || heads > 65535 || dv < 1)
+  if (!out || !partial_o || !partial_ml || !query_start_loc || splits < 1 || splits > FA_MAX_SPLITS || heads < 1 || heads > 65535 || dv < 1 ||
+      out_stride < (long)heads * dv)
     return TS_ERR_ARG;
   hipLaunchKernelGGL(attention_tiles_combine_kernel, dim3(items, heads), dim3(128), 0, stream, (uint16_t*)out,
-                     (const float*)partial_o, (const float*)partial_ml, query_start_loc, first_seq, heads, dv, splits, sinks, sink_scores);
+                     (const float*)partial_o, (const float*)partial_ml, query_start_loc, first_seq, heads, dv, splits, sinks, sink_scores,
+                     FaOut{out_stride, out_scale});
   return ts_launch_status();
 }

@@ -14,7 +14,7 @@
 // ---------------------------------------------------------------------------------------------
 template <typename T>
 __global__ void embed_kernel(float* __restrict__ residual, const T* __restrict__ table,
-                             const int* __restrict__ ids, int hidden, int vocab) {
+                             const int* __restrict__ ids, int hidden, int vocab, float scale) {
   const int t = blockIdx.x;
   int id = ids[t];
   const bool valid = id >= 0 && id < vocab;
@@ -22,19 +22,19 @@ __global__ void embed_kernel(float* __restrict__ residual, const T* __restrict__
   float* out = residual + (size_t)t * hidden;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
     // An id outside the table is a host error; it yields NaN instead of a read out of bounds.
-    out[i] = valid ? to_float(row[i]) : __uint_as_float(0x7fc00000u);
+    out[i] = valid ? to_float(row[i]) * scale : __uint_as_float(0x7fc00000u);
   }
 }
 
 extern "C" int ts_embed(void* residual, const void* table, const int* ids, int tokens, int hidden,
-                        int vocab, int dtype, hipStream_t stream) {
+                        int vocab, float scale, int dtype, hipStream_t stream) {
   if (tokens == 0) return TS_OK;
   if (!residual || !table || !ids || hidden < 1 || vocab < 1) return TS_ERR_ARG;
   dim3 grid(tokens), block(256);
   if (dtype == TS_F32)
-    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, (float*)residual, (const float*)table, ids, hidden, vocab);
+    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, (float*)residual, (const float*)table, ids, hidden, vocab, scale);
   else if (dtype == TS_BF16)
-    hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, (float*)residual, (const bf16_t*)table, ids, hidden, vocab);
+    hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, (float*)residual, (const bf16_t*)table, ids, hidden, vocab, scale);
   else
     return TS_ERR_DTYPE;
   return ts_launch_status();

@@ -175,10 +175,10 @@ gemm_tiled_kernel(float* __restrict__ partial, uint16_t* __restrict__ gated, con
       const int row = (SHARED_ROWS ? 0 : 16 * MB * wave_m) + 16 * b + lane16;
       if (row >= m) continue;
       if (gated) {
-        // The matrix is a gate|up projection with rows alternating gate, up (one range of K, no
-        // bias): the lane holds two such pairs and writes silu(gate) * up for both, rounded once,
+        // The matrix is a gate|up projection with rows alternating gate, up (one range of
+        // K): the lane holds two such pairs and writes silu(gate) * up for both, rounded once,
         // by the formula of the stand-alone SwiGLU kernel.
-        const f32x4 s = acc[a][b];
+        const f32x4 s = acc[a][b] + bv;
         const float lo = gated_unit(s[0], s[1], rule);
         const float hi = gated_unit(s[2], s[3], rule);
         uint16_t* out = gated + (size_t)row * (n / 2) + nrow / 2;
@@ -260,7 +260,7 @@ int launch_tiled_tall(float* partial, uint16_t* gated, const uint16_t* x, long x
 // or, for m <= 32, 8 (256 rows).
 // gated (bfloat16 [m, n / 2], contiguous) instead of partial: w is a gate|up projection whose rows
 // alternate gate, up, and the kernel writes the gated unit of the pair (silu(gate) * up for the rule
-// {1, 0, 0}); needs splits == 1, no bias, n even.
+// {1, 0, 0}); needs splits == 1, n even.
 extern "C" int ts_gemm_tiled(float* partial, void* gated, const void* x, long x_stride, const void* w,
                              const void* bias, int m, int n, int k, int iters_per_split, int splits, int tile,
                              float steepness, float limit, float up_shift, float cubic, hipStream_t stream) {
@@ -270,7 +270,7 @@ extern "C" int ts_gemm_tiled(float* partial, void* gated, const void* x, long x_
   const int total = (k + DEPTH - 1) / DEPTH;
   if (iters_per_split < 1 || splits != (total + iters_per_split - 1) / iters_per_split || splits > 65535)
     return TS_ERR_SHAPE;
-  if (gated && (splits != 1 || bias || (n & 1) != 0)) return TS_ERR_ARG;
+  if (gated && (splits != 1 || (n & 1) != 0)) return TS_ERR_ARG;
   const GluRule rule = {steepness, limit, up_shift, cubic};  // of the gated unit (common.hpp); {1, 0, 0}: silu(gate) * up
   uint16_t* gp = (uint16_t*)gated;
   const uint16_t* xp = (const uint16_t*)x;

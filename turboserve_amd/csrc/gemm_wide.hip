@@ -23,7 +23,7 @@
 //     weights then come from memory once and from that die's L2 afterwards.
 // Results: bfloat16 Y (one range of K; bias added), or 32-bit partial sums [S, M, N] over S
 // ranges of K (bias in the first; the consumer adds them up), or, for a gate|up matrix whose rows
-// alternate gate, up, silu(gate) * up as bfloat16 [M, N / 2] (one range of K, no bias).
+// alternate gate, up, silu(gate) * up as bfloat16 [M, N / 2] (one range of K).
 #include "common.hpp"
 
 namespace {
@@ -223,7 +223,7 @@ gemm_wide_kernel(float* __restrict__ partial, uint16_t* __restrict__ out, const 
       if (MODE == 2) {
         // rows of the matrix alternate gate, up: the lane holds two such pairs (the stand-alone
         // SwiGLU kernel's formula, rounded once)
-        const f32x4 s = acc[a][b];
+        const f32x4 s = acc[a][b] + bv;
         const float lo = gated_unit(s[0], s[1], rule);
         const float hi = gated_unit(s[2], s[3], rule);
         uint16_t* at = out + (size_t)row * (n / 2) + nrow / 2;
@@ -308,7 +308,7 @@ int launch_wide(int mode, float* partial, uint16_t* out, const uint16_t* x, long
 // x [m, k] bfloat16 with row stride x_stride; w [n, k] bfloat16 contiguous; bias [n] bfloat16 or
 // null; k % 8 == 0.  mode 0: out = bfloat16 [m, n] (splits must be 1); mode 1: partial = float
 // [splits, m, n]; mode 2: out = bfloat16 [m, n / 2] = silu(gate) * up for a w whose rows alternate
-// gate, up (splits 1, no bias, n even).  depth: k per iteration, 64 or (tiles of 64 activation rows
+// gate, up (splits 1, n even).  depth: k per iteration, 64 or (tiles of 64 activation rows
 // only) 128; iters_per_split iterations of `depth` of k go to each of `splits` =
 // ceil(ceil(k / depth) / iters_per_split) ranges.  tile: 2, 4, 5 or (with 8 wavefronts and 256 activation rows) 8 (64, 128, 160 or 256
 // weight rows a workgroup); x_rows: 128 or 256 (with 8 wavefronts also 64) activation rows a workgroup; waves: 4 or 8
@@ -324,7 +324,7 @@ extern "C" int ts_gemm_wide(float* partial, void* out, const void* x, long x_str
   const int total = (k + depth - 1) / depth;
   if (iters_per_split < 1 || splits != (total + iters_per_split - 1) / iters_per_split) return TS_ERR_SHAPE;
   if (mode != 1 && splits != 1) return TS_ERR_ARG;
-  if (mode == 2 && (bias || (n & 1) != 0)) return TS_ERR_ARG;
+  if (mode == 2 && (n & 1) != 0) return TS_ERR_ARG;
   const GluRule rule = {steepness, limit, up_shift, cubic};  // of mode 2's gated unit (common.hpp); {1, 0, 0}: silu(gate) * up
   uint16_t* op = (uint16_t*)out;
   const uint16_t* xp = (const uint16_t*)x;

@@ -6,7 +6,7 @@
 //     s = residual + p;  residual = s
 //     y = round_T(layer_norm(s) * w + b)             where a norm of the sum is given, else round_T(s)
 // with layer_norm(v) = (v - mean) / sqrt(variance + eps), the variance being the mean of the squared deviations
-// (two passes over registers), all in 32-bit with one rounding.  With `rows` the kernel reads rows[i] and writes
+// (two passes over registers), all in 32-bit with one rounding.  A norm without a bias has a null one.  With `rows` the kernel reads rows[i] and writes
 // y[i] only (residual untouched): the final norm at the wanted positions.  So one launch serves a block with a
 // norm in front of its parts, one with a norm behind them, and the head.
 //
@@ -16,7 +16,7 @@
 template <typename T>
 struct LayerNormRule {
   const T* w;  // null: no norm
-  const T* b;
+  const T* b;  // null: nothing is added
   float eps;
   float scale;
 };
@@ -46,7 +46,12 @@ __device__ __forceinline__ void ln_apply(float (&s)[CHUNKS][VEC], LayerNormRule<
     if (i < hidden) {
       float w[VEC], b[VEC];
       load_vec<T, VEC>(rule.w + i, w);
-      load_vec<T, VEC>(rule.b + i, b);
+      if (rule.b) {
+        load_vec<T, VEC>(rule.b + i, b);
+      } else {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) b[e] = 0.f;
+      }
 #pragma unroll
       for (int e = 0; e < VEC; ++e) s[c][e] = rule.scale * fmaf(s[c][e] * rstd, w[e], b[e]);
     }
@@ -143,7 +148,7 @@ extern "C" int ts_add_layer_norm(void* y, float* residual, const void* pending, 
                                  const void* b, float eps, const int* rows, int out_rows, int hidden, int dtype, hipStream_t stream) {
   if (out_rows == 0) return TS_OK;
   if (!y || !residual || hidden < 1 || splits < 1 || (splits > 1 && !pending) || (post_w && !pending)) return TS_ERR_ARG;
-  if ((post_w == nullptr) != (post_b == nullptr) || (w == nullptr) != (b == nullptr)) return TS_ERR_ARG;
+  if ((!post_w && post_b) || (!w && b)) return TS_ERR_ARG;
   if (dtype == TS_F32)
     return launch_add_layer_norm<float, float>(y, residual, pending, splits, split_stride, post_w, post_b, post_eps, post_scale, w, b, eps, rows, out_rows, hidden, stream);
   if (dtype == TS_BF16 && pending_f32)

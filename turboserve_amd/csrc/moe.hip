@@ -1,8 +1,8 @@
 // Routed feed-forward ("mixture of experts"): the router with its selection rule, the experts'
 // products for the (token, taken expert) pairs of a step, and the weighted sum.
 //
-// Router: z = R x comes from the engine's own product with a 32-bit result; here, all in 32-bit,
-// s = sigmoid(z), or softmax(z) over all the router's outputs.  Experts are chosen by c = s +
+// Router: z = R x comes from the engine's own product with a 32-bit result; here, all in 32-bit, a
+// bias per output is added where the router has one, then s = sigmoid(z), or softmax(z) over all the router's outputs.  Experts are chosen by c = s +
 // correction (a vector per layer; none: c = s).  The experts form `groups` equal groups of
 // neighbours; a group's mark is the sum of its two largest c (its one c if it has one member);
 // only experts of the `keep` groups with the largest marks can be taken; the `top` of them with
@@ -29,7 +29,8 @@ __device__ __forceinline__ int wave_argmax(float value, int index, float& best) 
 __global__ void __launch_bounds__(TS_WAVE)
 moe_select_kernel(int* __restrict__ taken, float* __restrict__ weights, float* __restrict__ extra_gate,
                   const float* __restrict__ z, int stride, int experts, int top, int groups, int keep,
-                  float route_scale, int softmax, const float* __restrict__ correction, int normalise, int mark_top) {
+                  float route_scale, int softmax, const float* __restrict__ correction, int normalise, int mark_top,
+                  const float* __restrict__ bias) {
   __shared__ float weight_of[MOE_MAX_EXPERTS];  // s: what a taken expert is weighted with
   __shared__ float score[MOE_MAX_EXPERTS];      // c: what experts are chosen by
   __shared__ float mark[MOE_MAX_EXPERTS];   // per group
@@ -39,18 +40,18 @@ moe_select_kernel(int* __restrict__ taken, float* __restrict__ weights, float* _
   const float* row = z + (size_t)t * stride;
   if (softmax) {
     float top_z = -INFINITY;
-    for (int e = lane; e < experts; e += TS_WAVE) top_z = fmaxf(top_z, row[e]);
+    for (int e = lane; e < experts; e += TS_WAVE) top_z = fmaxf(top_z, row[e] + (bias ? bias[e] : 0.f));
     top_z = wave_max(top_z);
     float sum = 0.f;
     for (int e = lane; e < experts; e += TS_WAVE) {
-      const float v = expf(row[e] - top_z);
+      const float v = expf(row[e] + (bias ? bias[e] : 0.f) - top_z);
       weight_of[e] = v;
       sum += v;
     }
     sum = wave_sum(sum);
     for (int e = lane; e < experts; e += TS_WAVE) weight_of[e] = weight_of[e] / sum;  // each lane its own entries
   } else {
-    for (int e = lane; e < experts; e += TS_WAVE) weight_of[e] = 1.f / (1.f + expf(-row[e]));
+    for (int e = lane; e < experts; e += TS_WAVE) weight_of[e] = 1.f / (1.f + expf(-(row[e] + (bias ? bias[e] : 0.f))));
   }
   for (int e = lane; e < experts; e += TS_WAVE) score[e] = weight_of[e] + (correction ? correction[e] : 0.f);
   if (extra_gate && lane == 0) extra_gate[t] = 1.f / (1.f + expf(-row[experts]));
@@ -108,14 +109,14 @@ moe_select_kernel(int* __restrict__ taken, float* __restrict__ weights, float* _
 
 extern "C" int ts_moe_select(int* taken, float* weights, float* extra_gate, const float* z, int tokens, int stride,
                              int experts, int top, int groups, int keep, float route_scale, int softmax,
-                             const float* correction, int normalise, int mark_top, hipStream_t stream) {
+                             const float* correction, int normalise, int mark_top, const float* bias, hipStream_t stream) {
   if (tokens == 0) return TS_OK;
   if (!taken || !weights || !z || mark_top < 1 || mark_top > 2) return TS_ERR_ARG;
   if (experts < 1 || experts > MOE_MAX_EXPERTS || top < 1 || top > MOE_MAX_TOP || groups < 1 || experts % groups != 0 ||
       keep < 1 || keep > groups || top > (experts / groups) * keep || stride < experts + (extra_gate ? 1 : 0))
     return TS_ERR_SHAPE;
   hipLaunchKernelGGL(moe_select_kernel, dim3(tokens), dim3(TS_WAVE), 0, stream, taken, weights, extra_gate, z, stride,
-                     experts, top, groups, keep, route_scale, softmax, correction, normalise, mark_top);
+                     experts, top, groups, keep, route_scale, softmax, correction, normalise, mark_top, bias);
   return ts_launch_status();
 }
 

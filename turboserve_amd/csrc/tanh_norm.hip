@@ -8,7 +8,7 @@
 // neighbouring elements (or one, where the row's size is no multiple of four) and a row may be
 // spread over several workgroups.
 //
-// ts_tanh_cap: x <- cap * tanh(x / cap) in place over 32-bit values.
+// ts_scale_cap: x <- scale * x, then, with a cap, x <- cap * tanh(x / cap), in place over 32-bit values.
 #include "common.hpp"
 
 template <typename P>
@@ -78,14 +78,16 @@ extern "C" int ts_add_tanh_norm(void* y, float* residual, const void* pending, i
   return ts_launch_status();
 }
 
-__global__ void __launch_bounds__(256) tanh_cap_kernel(float* __restrict__ x, size_t total, float cap) {
+__global__ void __launch_bounds__(256) scale_cap_kernel(float* __restrict__ x, size_t total, float scale, float cap) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < total) x[i] = cap * tanhf(x[i] / cap);
+  if (i >= total) return;
+  const float v = x[i] * scale;
+  x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
 }
 
-extern "C" int ts_tanh_cap(float* x, long total, float cap, hipStream_t stream) {
+extern "C" int ts_scale_cap(float* x, long total, float scale, float cap, hipStream_t stream) {
   if (total == 0) return TS_OK;
-  if (!x || !(cap > 0.f)) return TS_ERR_ARG;
-  hipLaunchKernelGGL(tanh_cap_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, x, (size_t)total, cap);
+  if (!x || !(cap >= 0.f)) return TS_ERR_ARG;
+  hipLaunchKernelGGL(scale_cap_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, x, (size_t)total, scale, cap);
   return ts_launch_status();
 }

@@ -37,7 +37,7 @@ MODULES: dict[str, tuple[str, ...]] = {
         "mixer_store.hip",
         "linear_state.hip",
         "delta_state.hip",
-        "selective_state.hip",
+        "decaying_state.hip",
         "short_conv.hip",
         "tanh_norm.hip",
         "layer_norm.hip",

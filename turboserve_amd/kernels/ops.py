@@ -57,7 +57,7 @@ def dtype_code(dtype: torch.dtype) -> int:
 
 _SIGNATURES: dict[str, dict[str, list]] = {
     "core": {
-        "ts_embed": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_embed": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_int, c_void_p],
         "ts_rmsnorm": [c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_float, c_int, c_int, c_void_p],
         "ts_add_rmsnorm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float,
                            c_int, c_int, c_float, c_int, c_int, c_void_p, c_int, c_long, c_void_p, c_float, c_float, c_void_p],
@@ -71,12 +71,12 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "ts_paged_attention_generic": [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int,
                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                        c_float, c_float, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_int,
-                                       c_void_p],
+                                       c_long, c_float, c_void_p],
         "ts_attention_tiles": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                                c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
-                               c_int, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
+                               c_int, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_float, c_void_p],
         "ts_attention_tiles_combine": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float,
-                                       c_void_p, c_void_p],
+                                       c_void_p, c_long, c_float, c_void_p],
         "ts_head_norm_store": [c_void_p, c_long, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_int, c_float, c_int,
@@ -92,16 +92,18 @@ _SIGNATURES: dict[str, dict[str, list]] = {
                            c_int, c_void_p],
         "ts_add_tanh_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float, c_void_p, c_int,
                              c_int, c_int, c_void_p, c_int, c_long, c_void_p],
-        "ts_tanh_cap": [c_void_p, c_long, c_float, c_void_p],
+        "ts_scale_cap": [c_void_p, c_long, c_float, c_float, c_void_p],
         "ts_short_conv": [c_void_p, c_int, c_void_p, c_int, c_int, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "ts_short_conv_carry": [c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                                 c_int, c_int, c_void_p],
-        "ts_selective_walk": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_void_p,
-                              c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
-        "ts_selective_pieces": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_void_p,
-                                c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
-        "ts_selective_carry": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+        "ts_decaying_walk": [*[c_void_p] * 6, c_int, c_int, c_long, *[c_int] * 4, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p,
+                             c_void_p, c_float, c_void_p, c_float, c_void_p, c_void_p, *[c_int] * 8, c_void_p],
+        "ts_decaying_pieces": [*[c_void_p] * 6, *[c_int] * 4, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_void_p, c_float,
+                               c_void_p, c_float, c_void_p, *[c_int] * 7, c_void_p],
+        "ts_decaying_carry": [*[c_void_p] * 8, *[c_int] * 5, c_void_p],
+        "ts_heads_finish": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_int, c_float,
+                            c_float, *[c_void_p] * 4, *[c_int] * 4, c_void_p],
         "ts_gated_group_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_int, c_void_p, c_float, c_int, c_int, c_int,
                                 c_int, c_void_p],
         "ts_add_layer_norm": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float, c_float, c_void_p,
@@ -127,7 +129,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "ts_copy_f32": [c_void_p, c_void_p, c_long, c_void_p],
         "ts_stream_offset": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
         "ts_moe_select": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                          c_int, c_void_p, c_int, c_int, c_void_p],
+                          c_int, c_void_p, c_int, c_int, c_void_p, c_void_p],
         "ts_moe_pair_rows": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                              c_float, c_float, c_float, c_int, c_void_p],
         "ts_moe_group": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
@@ -408,8 +410,8 @@ class Ops:
 
     # -- rows ---------------------------------------------------------------------------------
 
-    def embed(self, table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
-        """``float32 [T, H]`` rows of ``table [V, H]`` at ``ids [T]`` (the start of the 32-bit
+    def embed(self, table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor | None = None, *, scale: float = 1.0) -> torch.Tensor:
+        """``float32 [T, H]`` rows of ``table [V, H]`` at ``ids [T]``, times ``scale`` in 32-bit (the start of the 32-bit
         residual stream)."""
         _gpu(table, ids)
         _i32(ids, "ids")
@@ -419,7 +421,7 @@ class Ops:
             out = torch.empty((tokens, hidden), dtype=torch.float32, device=table.device)
         _need(out.shape == (tokens, hidden) and out.dtype == torch.float32 and out.is_contiguous(),
               "out must be contiguous float32 [T, H]")
-        _check(self.core.ts_embed(_ptr(out), _ptr(table), _ptr(ids), tokens, hidden, vocab,
+        _check(self.core.ts_embed(_ptr(out), _ptr(table), _ptr(ids), tokens, hidden, vocab, float(scale),
                                   dtype_code(table.dtype), self.stream()), "ts_embed")
         return out
 
@@ -1022,11 +1024,11 @@ class Ops:
                                           also_splits, also_stride, self.stream()), "ts_add_tanh_norm")
         return y
 
-    def tanh_cap(self, x: torch.Tensor, cap: float) -> torch.Tensor:
-        """``x <- cap * tanh(x / cap)`` in place over a contiguous 32-bit tensor."""
+    def scale_cap(self, x: torch.Tensor, *, scale: float = 1.0, cap: float = 0.0) -> torch.Tensor:
+        """``x <- scale * x`` and then, with a ``cap``, ``x <- cap * tanh(x / cap)``, in place over a contiguous 32-bit tensor."""
         _gpu(x)
-        _need(x.dtype == torch.float32 and x.is_contiguous() and cap > 0.0, "a positive cap on contiguous float32 values")
-        _check(self.core.ts_tanh_cap(_ptr(x), x.numel(), float(cap), self.stream()), "ts_tanh_cap")
+        _need(x.dtype == torch.float32 and x.is_contiguous() and cap >= 0.0, "contiguous float32 values, and a cap that is not negative")
+        _check(self.core.ts_scale_cap(_ptr(x), x.numel(), float(scale), float(cap), self.stream()), "ts_scale_cap")
         return x
 
     def short_conv(self, proj: torch.Tensor, first_col: int, taps: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor,
@@ -1127,12 +1129,12 @@ class Ops:
     # -- layer norm, two-table embedding ---------------------------------------------------------
 
     def add_layer_norm(self, residual: torch.Tensor, pending: torch.Tensor | None, dtype: torch.dtype, rows: torch.Tensor | None = None, *,
-                       norm: tuple[torch.Tensor, torch.Tensor, float] | None = None,
-                       pending_norm: tuple[torch.Tensor, torch.Tensor, float, float] | None = None) -> torch.Tensor:
+                       norm: tuple[torch.Tensor, torch.Tensor | None, float] | None = None,
+                       pending_norm: tuple[torch.Tensor, torch.Tensor | None, float, float] | None = None) -> torch.Tensor:
         """``residual += p`` in 32-bit (in place) and the sum in ``dtype``, rounded once: through a layer norm where
         ``norm = (weight [H], bias [H], eps)`` is given, as it is otherwise.  ``p`` is ``pending`` (``[T, H]`` of
         ``dtype`` or ``[S, T, H]`` 32-bit partial sums), with ``pending_norm = (weight, bias, eps, scale)`` first
-        normalised on its own and multiplied by ``scale``, in 32-bit.  With ``rows`` only those rows, and ``residual`` is left
+        normalised on its own and multiplied by ``scale``, in 32-bit.  A bias may be ``None``: nothing is added.  With ``rows`` only those rows, and ``residual`` is left
         alone."""
         _gpu(residual, pending, rows)
         _i32(rows, "rows")
@@ -1147,7 +1149,7 @@ class Ops:
         for rule in (norm, pending_norm):
             for t in () if rule is None else rule[:2]:
                 _gpu(t)
-                _need(t.shape == (hidden,) and t.dtype == dtype and t.is_contiguous(), "a layer norm's weight and bias must be [H] of the run dtype")
+                _need(t is None and t is not rule[0] or t.shape == (hidden,) and t.dtype == dtype and t.is_contiguous(), "a layer norm's weight and bias must be [H] of the run dtype")
         w, b, eps = (None, None, 0.0) if norm is None else norm
         post_w, post_b, post_eps, post_scale = (None, None, 0.0, 1.0) if pending_norm is None else pending_norm
         out_rows = tokens if rows is None else rows.numel()
@@ -1177,63 +1179,155 @@ class Ops:
                                          int(mul_cur) % buckets, dtype_code(table.dtype), self.stream()), "ts_embed_bigram")
         return out
 
-    # -- a selective state space -----------------------------------------------------------------
+    # -- states that decay by one number per head and token ------------------------------------------
 
     #: Tokens of a piece when long portions are cut up to run side by side (the kernels' own constant).
-    selective_piece = 128
+    decaying_piece = 128
     #: Portions of up to this many tokens are walked, longer ones (bfloat16 runs) cut into pieces.
-    selective_walk_tokens = 32
+    decaying_walk_tokens = 32
 
     @staticmethod
-    def selective_pieces_supported(dtype: torch.dtype, state_dim: int, value_dim: int) -> bool:
+    def decaying_pieces_supported(dtype: torch.dtype, state_dim: int, value_dim: int) -> bool:
         """Whether long portions can be cut into pieces on the matrix cores: bfloat16, state rows of up to 256,
         state rows and columns both multiples of 8 (16-byte accesses)."""
         return dtype == torch.bfloat16 and state_dim <= 256 and state_dim % 8 == 0 and value_dim % 8 == 0
 
-    def selective_state(self, u: torch.Tensor, proj: torch.Tensor, dt_at: int, dt_bias: torch.Tensor, a_log: torch.Tensor,
-                        skip: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, query_start_loc: torch.Tensor, *,
-                        num_seqs: int, heads: int, groups: int, state_dim: int, value_dim: int, dtype: torch.dtype,
-                        plan: tuple | None = None) -> torch.Tensor:
-        """A selective state space over a step: per head and request a 32-bit state ``S [N, P]`` (``state [slots, H, P,
-        N]``) that every token decays and adds to: ``dt = softplus(d + dt_bias)``, ``S <- exp(-exp(a_log) dt) S + dt B
-        x^T``, ``y = S^T C + skip x``.  ``u [T, H P + 2 G N]`` of ``dtype`` holds the step's convolved ``x | B | C`` (head
-        ``h`` uses group ``h // (H / G)``), ``d`` is the ``H`` columns of ``proj`` from ``dt_at`` on.  Returns ``y [T, H P]``
-        32-bit.  Without a ``plan`` every request is walked; ``plan = (pieces, carries, n_pieces, n_requests)`` (int32
-        device tensors from :meth:`linear_state_pieces`, for the requests from 0 on) cuts the first ``n_requests`` into
-        pieces of :attr:`selective_piece` tokens that run side by side, and the requests behind them are walked."""
-        _gpu(u, proj, dt_bias, a_log, skip, state, state_slots, query_start_loc)
+    def decaying_plan(self, ctx, dtype: torch.dtype, state_dim: int, value_dim: int) -> tuple | None:
+        """What :meth:`decaying_state` cuts a step's long portions by (made once per step, shared by the layers), or
+        ``None`` where every request is walked."""
+        if ctx.recorded or ctx.max_query_len <= self.decaying_walk_tokens or not self.decaying_pieces_supported(dtype, state_dim, value_dim):
+            return None
+
+        def cut(step) -> tuple:  # the requests that bring several tokens come first
+            pieces, carries = self.linear_state_pieces(step.query_lens[: step.num_prefill_seqs], self.decaying_piece)
+            both = self.device_ints(pieces + carries)
+            return both[: len(pieces)], both[len(pieces):], len(pieces), len(carries)
+
+        return ctx.derive(("decaying_pieces", self.decaying_piece), cut)
+
+    def decaying_state(self, rule: str, u: torch.Tensor, columns: tuple[int, int, int], state: torch.Tensor, state_slots: torch.Tensor,
+                       query_start_loc: torch.Tensor, *, num_seqs: int, heads: int, groups: int, state_dim: int, value_dim: int,
+                       dtype: torch.dtype, proj: torch.Tensor | None = None, first_gate: int = 0, numbers: tuple = (None, None),
+                       cap: float = 0.0, skip: torch.Tensor | None = None, scale: float = 1.0, sums: torch.Tensor | None = None,
+                       tops: torch.Tensor | None = None, plan: tuple | None = None) -> tuple[torch.Tensor, torch.Tensor | None]:
+        """A state that decays by one number per head and token, over a step: per head and request a 32-bit ``S [N, P]``
+        (``state [slots, H, P, N]``), ``S <- a S + w B x^T``, ``y = scale S^T C``.  A row of ``u [T, W]`` (of ``dtype``, or 32-bit
+        partial sums ``[S, T, W]``) holds ``x`` of ``H P``, ``B`` and ``C`` of ``G N`` columns, from ``columns = (x, B, C)`` on
+        (head ``h`` uses group ``h // (H / G)``).  ``rule``:
+
+        * ``"selective"``: ``dt = softplus(d + numbers[0])``, ``a = exp(-exp(numbers[1]) dt)``, ``w = dt``, ``d`` the ``H`` columns of
+          ``proj`` from ``first_gate`` on; ``y`` gets ``skip x`` added.
+        * ``"fixed"``: ``a = numbers[0]``, ``w = 1``.
+        * ``"gated"``: ``i = cap tanh((i' + numbers[0]) / cap)``, ``f = log sigmoid(cap tanh((f' + numbers[1]) / cap))``, ``i'`` and ``f'``
+          the ``2 H`` columns of ``proj`` from ``first_gate`` on; with a running maximum ``m`` (``tops [slots, H]``) ``m' = max(f +
+          m, i)``, ``a = exp(f + m - m')``, ``w = exp(i - m')``; a sum ``n [N]`` (``sums [slots, H, N]``) takes ``a n + w B``.  The
+          slots' ``m`` is read only: :meth:`heads_finish` moves it on.
+
+        All in 32-bit; ``numbers`` are 32-bit ``[H]``.  Returns ``(y [T, H P], norm)``, both 32-bit, ``norm [T, H, 2]`` being ``(scale
+        n . C, m')`` for the gated rule, else ``None``.  Without a ``plan`` every request is walked; ``plan = (pieces, carries,
+        n_pieces, n_requests)`` (:meth:`decaying_plan`) cuts the first ``n_requests`` into pieces of :attr:`decaying_piece` tokens
+        that run side by side, and the requests behind them are walked."""
+        _gpu(u, state, state_slots, query_start_loc, proj, skip, sums, tops, *numbers)
         _i32(state_slots, "state_slots")
         _i32(query_start_loc, "query_start_loc")
-        tokens, width = proj.shape[-2], proj.shape[-1]
-        is_f32, splits, stride = self._partials(proj, tokens, width, dtype, "projection")
-        _need(u.dtype == dtype and u.is_contiguous() and u.shape == (tokens, heads * value_dim + 2 * groups * state_dim),
-              "the convolved x | B | C must be [T, H P + 2 G N] of the run dtype")
-        _need(heads % groups == 0 and 1 <= state_dim <= 512 and 0 <= dt_at and dt_at + heads <= width, "sizes the selective state does not take")
-        for t in (dt_bias, a_log, skip):
-            _need(t.shape == (heads,) and t.dtype == torch.float32 and t.is_contiguous(), "dt_bias, a_log and skip must be float32 [H]")
+        code = {"selective": 0, "fixed": 1, "gated": 2}[rule]
+        tokens, u_width = u.shape[-2], u.shape[-1]
+        u_f32, u_splits, u_stride = self._partials(u, tokens, u_width, dtype, "the vectors' rows")
+        is_f32, splits, stride, width = 0, 1, 0, 0
+        if code != 1:
+            _need(proj is not None, "this rule reads the projection")
+            width = proj.shape[-1]
+            is_f32, splits, stride = self._partials(proj, tokens, width, dtype, "projection")
+        _need(heads % groups == 0 and 1 <= state_dim <= 512 and 1 <= value_dim <= 65534, "sizes the decaying state does not take")
+        for at, size in zip(columns, (heads * value_dim, groups * state_dim, groups * state_dim)):
+            _need(0 <= at and at + size <= u_width, "the vectors' columns must lie inside the rows")
+        _need(0 <= first_gate and (code == 1 or first_gate + (2 if code == 2 else 1) * heads <= width), "the gates' columns must lie inside the projection")
+        wanted = {0: (*numbers, skip), 1: numbers[:1], 2: numbers}[code]
+        for t in wanted:
+            _need(t is not None and t.shape == (heads,) and t.dtype == torch.float32 and t.is_contiguous(), "a rule's numbers must be float32 [H]")
         _need(state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (heads, value_dim, state_dim),
               "the state must be float32 [slots, H, P, N]")
         _need(query_start_loc.numel() >= num_seqs + 1 and state_slots.numel() >= num_seqs, "row ranges and slots of every request")
+        norm = None
+        if code == 2:
+            _need(cap > 0.0 and sums is not None and tops is not None and sums.dtype == tops.dtype == torch.float32 and sums.is_contiguous()
+                  and tops.is_contiguous() and sums.shape == (state.shape[0], heads, state_dim) and tops.shape == (state.shape[0], heads),
+                  "sums [slots, H, N] and tops [slots, H] must be float32, and the cap positive")
+            norm = torch.empty((tokens, heads, 2), dtype=torch.float32, device=u.device)
         y = torch.empty((tokens, heads * value_dim), dtype=torch.float32, device=u.device)
-        steps = (_ptr(proj), is_f32, splits, stride, width, dt_at, _ptr(dt_bias), _ptr(a_log), _ptr(skip))
+        rows = (u_width, *(int(c) for c in columns))
+        gates = (_ptr(proj), is_f32, splits, stride, width, int(first_gate), _ptr(numbers[0]), _ptr(numbers[1]) if len(numbers) > 1 else None,
+                 float(cap), _ptr(skip), float(scale))
         first = 0
         if plan is not None:
             pieces, carries, n_pieces, first = plan
             _i32(pieces, "pieces")
             _i32(carries, "carries")
-            _need(self.selective_pieces_supported(dtype, state_dim, value_dim) and first <= num_seqs, "a geometry that is not cut into pieces")
-            piece_state = torch.empty((n_pieces, heads, value_dim, state_dim), dtype=torch.float32, device=u.device)
-            piece_decay = torch.empty((n_pieces, heads), dtype=torch.float32, device=u.device)
+            _need(self.decaying_pieces_supported(dtype, state_dim, value_dim) and first <= num_seqs, "a geometry that is not cut into pieces")
+            rounded = u if u.dim() == 2 else self.dense(u, dtype)
+            held = value_dim + (1 if code == 2 else 0)
+            piece_state = torch.empty((n_pieces, heads, held, state_dim), dtype=torch.float32, device=u.device)
+            piece_decay = torch.empty((n_pieces, heads, 2), dtype=torch.float32, device=u.device)
+            piece_top = torch.empty((n_pieces, heads), dtype=torch.float32, device=u.device) if code == 2 else None
             for mode in (0, 1):
-                _check(self.core.ts_selective_pieces(_ptr(y), _ptr(piece_state), _ptr(piece_decay), _ptr(u), *steps, _ptr(pieces), n_pieces,
-                                                     heads, groups, state_dim, value_dim, mode, self.stream()), "ts_selective_pieces")
+                _check(self.core.ts_decaying_pieces(
+                    _ptr(y), _ptr(norm), _ptr(piece_state), _ptr(piece_decay), _ptr(piece_top), _ptr(rounded), *rows, *gates, _ptr(pieces),
+                    n_pieces, heads, groups, state_dim, value_dim, code, mode, self.stream()), "ts_decaying_pieces")
                 if mode == 0:
-                    _check(self.core.ts_selective_carry(_ptr(state), _ptr(state_slots), _ptr(carries), _ptr(piece_state), _ptr(piece_decay),
-                                                        first, heads, state_dim, value_dim, self.stream()), "ts_selective_carry")
-        _check(self.core.ts_selective_walk(_ptr(y), _ptr(state), _ptr(u), 1 if dtype == torch.float32 else 0, *steps, _ptr(state_slots),
-                                           _ptr(query_start_loc), first, num_seqs - first, heads, groups, state_dim, value_dim,
-                                           dtype_code(dtype), self.stream()), "ts_selective_walk")
+                    _check(self.core.ts_decaying_carry(
+                        _ptr(state), _ptr(sums), _ptr(tops), _ptr(state_slots), _ptr(carries), _ptr(piece_state), _ptr(piece_decay),
+                        _ptr(piece_top), first, heads, state_dim, value_dim, code, self.stream()), "ts_decaying_carry")
+        _check(self.core.ts_decaying_walk(
+            _ptr(y), _ptr(norm), _ptr(state), _ptr(sums), _ptr(tops), _ptr(u), 1 if u_f32 or dtype == torch.float32 else 0, u_splits, u_stride,
+            *rows, *gates, _ptr(state_slots), _ptr(query_start_loc), first, num_seqs - first, heads, groups, state_dim, value_dim, code,
+            dtype_code(dtype), self.stream()), "ts_decaying_walk")
+        return y, norm
+
+    def selective_state(self, u: torch.Tensor, proj: torch.Tensor, dt_at: int, dt_bias: torch.Tensor, a_log: torch.Tensor,
+                        skip: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, query_start_loc: torch.Tensor, *,
+                        num_seqs: int, heads: int, groups: int, state_dim: int, value_dim: int, dtype: torch.dtype,
+                        plan: tuple | None = None) -> torch.Tensor:
+        """A selective state space over a step (:meth:`decaying_state`): ``u [T, H P + 2 G N]`` of ``dtype`` holds the step's
+        convolved ``x | B | C``, ``d`` is the ``H`` columns of ``proj`` from ``dt_at`` on.  Returns ``y [T, H P]`` 32-bit."""
+        inner = heads * value_dim
+        _need(u.dtype == dtype and u.is_contiguous() and u.shape == (proj.shape[-2], inner + 2 * groups * state_dim),
+              "the convolved x | B | C must be [T, H P + 2 G N] of the run dtype")
+        y, _ = self.decaying_state(
+            "selective", u, (0, inner, inner + groups * state_dim), state, state_slots, query_start_loc, num_seqs=num_seqs, heads=heads,
+            groups=groups, state_dim=state_dim, value_dim=value_dim, dtype=dtype, proj=proj, first_gate=dt_at, numbers=(dt_bias, a_log),
+            skip=skip, plan=plan)
         return y
+
+    def heads_finish(self, y: torch.Tensor, proj: torch.Tensor, gate_at: int, heads: int, eps: float, dtype: torch.dtype, *,
+                     gate: str = "silu", gain: torch.Tensor | None = None, norm: torch.Tensor | None = None,
+                     tops: torch.Tensor | None = None, state_slots: torch.Tensor | None = None, token_seq: torch.Tensor | None = None,
+                     query_start_loc: torch.Tensor | None = None, scale: float = 1.0,
+                     out: tuple[torch.Tensor, int] | None = None) -> torch.Tensor:
+        """``[T, H P]`` of ``dtype``: every head of the 32-bit ``y [T, H P]`` divided by its root mean square (``eps`` inside
+        the root), times ``gain [H P]`` where given, times ``silu`` or ``sigmoid`` (``gate``) of the ``H P`` columns of ``proj``
+        from ``gate_at`` on, times ``scale``, in 32-bit with one rounding.  With ``norm [T, H, 2]`` (a sum ``s`` and a running
+        maximum ``m`` per token and head, :meth:`decaying_state`) a head is first divided by ``max(|s|, exp(-m)) + 1e-6``, and
+        ``m`` of each request's last token is left in the request's slot of ``tops [slots, H]``.  ``out = (buffer, col0)``: the
+        result is written into those columns of a wider buffer, which is returned."""
+        _gpu(y, proj, gain, norm, tops, state_slots, token_seq, query_start_loc)
+        tokens, width = y.shape
+        is_f32, splits, stride = self._partials(proj, tokens, proj.shape[-1], dtype, "projection")
+        _need(y.dtype == torch.float32 and y.is_contiguous() and width % heads == 0, "y must be float32 [T, H P]")
+        _need(gate in ("silu", "sigmoid") and 0 <= gate_at and gate_at + width <= proj.shape[-1], "the gate's columns must lie inside the projection")
+        _need(gain is None or (gain.shape == (width,) and gain.dtype == dtype and gain.is_contiguous()), "the gain must be [H P] of the run dtype")
+        if norm is not None:
+            for t, what in ((state_slots, "state_slots"), (token_seq, "token_seq"), (query_start_loc, "query_start_loc")):
+                _need(t is not None, "moving the maxima on needs the requests' rows and slots")
+                _i32(t, what)
+            _need(norm.dtype == torch.float32 and norm.is_contiguous() and norm.shape == (tokens, heads, 2) and tops is not None
+                  and tops.dtype == torch.float32 and tops.is_contiguous() and tops.shape[1:] == (heads,) and token_seq.numel() >= tokens,
+                  "norm [T, H, 2] and tops [slots, H] must be float32")
+        result, pointer, out_stride = self._columns_of(out, tokens, width, dtype, y.device)
+        _check(self.core.ts_heads_finish(
+            pointer, out_stride, _ptr(y), _ptr(norm), _ptr(proj), is_f32, splits, stride, proj.shape[-1], int(gate_at), _ptr(gain),
+            1 if gate == "sigmoid" else 0, float(eps), float(scale), _ptr(tops), _ptr(state_slots), _ptr(token_seq), _ptr(query_start_loc),
+            tokens, heads, width // heads, dtype_code(dtype), self.stream()), "ts_heads_finish")
+        return result
 
     def gated_group_norm(self, y: torch.Tensor, proj: torch.Tensor, z_at: int, gain: torch.Tensor, eps: float, parts: int,
                          dtype: torch.dtype) -> torch.Tensor:
@@ -1255,9 +1349,10 @@ class Ops:
 
     def moe_route(self, x: torch.Tensor, router: torch.Tensor, *, top: int, groups: int, keep: int, scale: float,
                   experts: int | None = None, softmax: bool = False, correction: torch.Tensor | None = None,
-                  normalise: bool = True, mark_top: int = 2) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
+                  normalise: bool = True, mark_top: int = 2,
+                  bias: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
         """The router of a routed feed-forward: ``z = x router^T`` by the engine's product with a
-        32-bit result, then in 32-bit ``s = sigmoid(z)`` or, with ``softmax``, the softmax over the
+        32-bit result, plus ``bias [experts]`` (32-bit) where given, then in 32-bit ``s = sigmoid(z)`` or, with ``softmax``, the softmax over the
         ``experts`` outputs; experts are chosen by ``c = s + correction`` (``correction [experts]``
         32-bit; none: ``c = s``): they form ``groups`` equal groups of neighbours, a group's mark is
         the sum of its two largest ``c`` (``mark_top = 1``: its largest alone), only the ``keep`` best groups' experts can be taken, the
@@ -1265,7 +1360,7 @@ class Ops:
         float32, gate)``: weights are ``s / (sum of the taken s + 1e-20) * scale``, or ``s * scale``
         where ``normalise`` is off.  With ``experts`` one less than the rows of ``router``, the last
         row is a gate's vector and ``gate [T]`` the sigmoid of its product (else ``None``)."""
-        _gpu(x, router, correction)
+        _gpu(x, router, correction, bias)
         _need(x.dim() == 2 and x.is_contiguous() and router.dim() == 2 and router.is_contiguous()
               and router.shape[1] == x.shape[1] and router.dtype == x.dtype, "x [T, H] and router [E, H] of one dtype")
         tokens = x.shape[0]
@@ -1276,6 +1371,9 @@ class Ops:
         if correction is not None:
             _need(correction.shape == (experts,) and correction.dtype == torch.float32 and correction.is_contiguous(),
                   "the correction must be contiguous float32 [experts]")
+        if bias is not None:
+            _need(bias.shape == (experts,) and bias.dtype == torch.float32 and bias.is_contiguous(),
+                  "the router's bias must be contiguous float32 [experts]")
         z = self.linear_float32_out(x, router)
         _need(z.dtype == torch.float32 and z.stride(1) == 1, "the router's outputs must be 32-bit rows")
         taken = torch.empty((tokens, top), dtype=torch.int32, device=x.device)
@@ -1283,7 +1381,7 @@ class Ops:
         gate = torch.empty((tokens,), dtype=torch.float32, device=x.device) if router.shape[0] > experts else None
         _check(self.core.ts_moe_select(_ptr(taken), _ptr(weights), _ptr(gate), _ptr(z), tokens, z.stride(0), experts, top,
                                        groups, keep, float(scale), 1 if softmax else 0, _ptr(correction),
-                                       1 if normalise else 0, int(mark_top), self.stream()), "ts_moe_select")
+                                       1 if normalise else 0, int(mark_top), _ptr(bias), self.stream()), "ts_moe_select")
         return taken, weights, gate
 
     def moe_pair_rows(self, rows: torch.Tensor, weight: torch.Tensor, taken: torch.Tensor | None, *, share: int,
@@ -1447,6 +1545,8 @@ class Ops:
         sink_scores: torch.Tensor | None = None,
         distance_bias: torch.Tensor | None = None,
         keep_first: int = 0,
+        out_scale: float = 1.0,
+        out: tuple[torch.Tensor, int] | None = None,
     ) -> torch.Tensor:
         """Attention of every token over the keys ``lo..position`` of its request (behind a window
         also over the request's first ``keep_first`` keys).  With
@@ -1460,7 +1560,8 @@ class Ops:
         counts ``n`` more keys of score 0 that have no value.  ``v_pages = None`` with ``value_dim =
         Dv <= D``: a key's value is its own first ``Dv`` elements.  ``sink_scores [heads]`` (32-bit):
         the sinks' score per head instead of 0.  ``distance_bias [heads, L]`` (32-bit): the score of
-        the key ``n`` positions back gets ``distance_bias[h, min(n, L - 1)]`` added."""
+        the key ``n`` positions back gets ``distance_bias[h, min(n, L - 1)]`` added.  The result is multiplied by
+        ``out_scale``; ``out = (buffer, col0)``: it is written into those columns of a wider buffer, which is returned."""
         _gpu(q, k_pages, v_pages, block_table, token_seq, positions)
         self._score_tables(heads, sinks, sink_scores, distance_bias)
         if slopes is not None:
@@ -1487,15 +1588,15 @@ class Ops:
         _need(block_table.dim() == 2 and token_seq.numel() == tokens, "block_table [S, MB], token_seq [T]")
         _need(1 <= kv_heads and heads % kv_heads == 0 and heads <= 65535 and 1 <= head_dim <= ATTENTION_MAX_ROW,
               f"{heads} query heads on {kv_heads} KV heads of {head_dim} elements are outside what the kernel takes")
-        out = self.rows_buffer(tokens, heads * value_dim, q.dtype, q.device)
+        result, pointer, out_stride = self._columns_of(out, tokens, heads * value_dim, q.dtype, q.device)
         _check(self.core.ts_paged_attention_generic(
-            _ptr(out), _ptr(q), q_stride, _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
+            pointer, _ptr(q), q_stride, _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
             block_table.shape[1], _ptr(token_seq), _ptr(positions), tokens, heads, kv_heads, head_dim, value_dim,
             block_size, float(scale), float(softcap), int(window or 0), _ptr(slopes) if slopes is not None else None,
             int(chunk or 0), float(sinks), _ptr(sink_scores), _ptr(distance_bias),
-            0 if distance_bias is None else distance_bias.shape[1], int(keep_first), dtype_code(q.dtype), self.stream()),
-            "ts_paged_attention_generic")
-        return out
+            0 if distance_bias is None else distance_bias.shape[1], int(keep_first), dtype_code(q.dtype), out_stride, float(out_scale),
+            self.stream()), "ts_paged_attention_generic")
+        return result
 
     @staticmethod
     def _score_tables(heads: int, sinks: float, sink_scores: torch.Tensor | None, distance_bias: torch.Tensor | None) -> None:
@@ -1544,13 +1645,15 @@ class Ops:
                         num_decode_seqs: int, max_decode_context: int, window: int | None = None, chunk: int | None = None,
                         sinks: float = 0.0, slopes: torch.Tensor | None = None, softcap: float = 0.0,
                         value_dim: int | None = None, sink_scores: torch.Tensor | None = None,
-                        distance_bias: torch.Tensor | None = None, keep_first: int = 0) -> torch.Tensor:
+                        distance_bias: torch.Tensor | None = None, keep_first: int = 0, out_scale: float = 1.0,
+                        out: tuple[torch.Tensor, int] | None = None) -> torch.Tensor:
         """What :meth:`paged_attention_generic` computes, for bfloat16, on the matrix cores: the
         requests that bring several tokens (the first ``num_prefill_seqs``) in tiles of 64 tokens by
         one head (``prefill_tiles``: int32 ``[n, 2]`` from :meth:`attention_tile_list`), the
         ``num_decode_seqs`` single tokens behind them with the heads of a KV head as one tile and
         their keys (at most ``max_decode_context``, a bound the step's shape gives) shared out over
-        several workgroups.  Returns ``[T, heads * Dv]``."""
+        several workgroups.  Returns ``[T, heads * Dv]``, times ``out_scale``; ``out = (buffer, col0)``: written into those
+        columns of a wider buffer, which is returned."""
         _gpu(q, k_pages, v_pages, block_table, query_start_loc, context_lens, prefill_tiles, slopes)
         self._score_tables(heads, sinks, sink_scores, distance_bias)
         tables = (_ptr(sink_scores), _ptr(distance_bias), 0 if distance_bias is None else distance_bias.shape[1], int(keep_first))
@@ -1573,14 +1676,15 @@ class Ops:
         _need(block_table.dim() == 2 and query_start_loc.numel() >= num_prefill_seqs + num_decode_seqs + 1, "block_table [S, MB], row ranges [S + 1]")
         if slopes is not None:
             _need(slopes.dtype == torch.float32 and slopes.is_contiguous() and slopes.numel() == heads, "slopes must be float32 [heads]")
-        out = self.rows_buffer(tokens, heads * value_dim, q.dtype, q.device)
+        result, pointer, out_stride = self._columns_of(out, tokens, heads * value_dim, q.dtype, q.device)
+        placed = (out_stride, float(out_scale))
         common = (_ptr(q), q_stride, _ptr(k_pages), _ptr(v_pages), _ptr(block_table), block_table.shape[1],
                   _ptr(query_start_loc), _ptr(context_lens))
         rule = (float(scale), float(softcap), int(window or 0), int(chunk or 0), float(sinks), _ptr(slopes))
         if num_prefill_seqs > 0:
             _need(prefill_tiles is not None and prefill_tiles.dim() == 2 and prefill_tiles.shape[1] == 2, "prefill_tiles [n, 2]")
-            _check(self.core.ts_attention_tiles(_ptr(out), None, None, *common, _ptr(prefill_tiles), prefill_tiles.shape[0], 0,
-                                                heads, kv_heads, head_dim, value_dim, block_size, *rule, 0, 1, *tables, self.stream()),
+            _check(self.core.ts_attention_tiles(pointer, None, None, *common, _ptr(prefill_tiles), prefill_tiles.shape[0], 0,
+                                                heads, kv_heads, head_dim, value_dim, block_size, *rule, 0, 1, *tables, *placed, self.stream()),
                    "ts_attention_tiles")
         if num_decode_seqs > 0:
             # Workgroups per (request, KV head): enough to fill the compute units (key rows of up to 128
@@ -1597,15 +1701,15 @@ class Ops:
             if splits > 1:
                 partial_o = torch.empty((num_decode_seqs, heads, splits, value_dim), dtype=torch.float32, device=q.device)
                 partial_ml = torch.empty((num_decode_seqs, heads, splits, 2), dtype=torch.float32, device=q.device)
-            _check(self.core.ts_attention_tiles(_ptr(out), _ptr(partial_o), _ptr(partial_ml), *common, None, num_decode_seqs,
+            _check(self.core.ts_attention_tiles(pointer, _ptr(partial_o), _ptr(partial_ml), *common, None, num_decode_seqs,
                                                 num_prefill_seqs, heads, kv_heads, head_dim, value_dim, block_size, *rule, 1,
-                                                splits, *tables, self.stream()), "ts_attention_tiles")
+                                                splits, *tables, *placed, self.stream()), "ts_attention_tiles")
             if splits > 1:
-                _check(self.core.ts_attention_tiles_combine(_ptr(out), _ptr(partial_o), _ptr(partial_ml), _ptr(query_start_loc),
+                _check(self.core.ts_attention_tiles_combine(pointer, _ptr(partial_o), _ptr(partial_ml), _ptr(query_start_loc),
                                                             num_decode_seqs, num_prefill_seqs, heads, value_dim, splits,
-                                                            float(sinks), _ptr(sink_scores), self.stream()),
+                                                            float(sinks), _ptr(sink_scores), *placed, self.stream()),
                        "ts_attention_tiles_combine")
-        return out
+        return result
 
     @staticmethod
     def mfma_attention_supported(dtype: torch.dtype, head_dim: int, block_size: int) -> bool:
@@ -1926,10 +2030,9 @@ class Ops:
         per_split, splits, tile = plan or self._tiled_plan(m, n, k, max_splits)
         x_stride = x.stride(0) if m > 1 else max(k, x.stride(0))
         if gated:
-            _need(splits == 1 and bias is None and n % 2 == 0,
-                  "the gated result needs one range of K, no bias and an even number of weight rows")
+            _need(splits == 1 and n % 2 == 0, "the gated result needs one range of K and an even number of weight rows")
             out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
-            _check(self.core.ts_gemm_tiled(None, _ptr(out), _ptr(x), x_stride, _ptr(weight), None, m, n, k,
+            _check(self.core.ts_gemm_tiled(None, _ptr(out), _ptr(x), x_stride, _ptr(weight), _ptr(bias), m, n, k,
                                            per_split, splits, tile, *glu_rule(rule), self.stream()),
                    "ts_gemm_tiled")
             return out
@@ -2036,7 +2139,7 @@ class Ops:
         of K, ranges, tile, activation rows a workgroup, wavefronts a workgroup[, k per iteration: 64 (the default) or 128]).  One range: bfloat16 ``[M, N]``; several
         (or, with ``sums``, one as well): 32-bit partial sums ``[S, M, N]`` (bias in the first).  ``gated``: the weight is a gate|up
         projection whose rows alternate gate, up, and the result is ``silu(gate) * up`` as
-        bfloat16 ``[M, N / 2]`` (one range of K, no bias)."""
+        bfloat16 ``[M, N / 2]`` (one range of K)."""
         _gpu(x, weight, bias)
         _need(x.dim() == 2 and x.stride(1) == 1 and weight.dim() == 2 and weight.is_contiguous()
               and x.shape[1] == weight.shape[1], "x must be [M, K] with unit inner stride, weight contiguous [N, K]")
@@ -2050,10 +2153,9 @@ class Ops:
         depth = plan[5] if len(plan) > 5 else 64
         x_stride = x.stride(0) if m > 1 else max(k, x.stride(0))
         if gated:
-            _need(splits == 1 and bias is None and n % 2 == 0,
-                  "the gated result needs one range of K, no bias and an even number of weight rows")
+            _need(splits == 1 and n % 2 == 0, "the gated result needs one range of K and an even number of weight rows")
             out = self.rows_buffer(m, n // 2, torch.bfloat16, x.device)
-            _check(self.core.ts_gemm_wide(None, _ptr(out), _ptr(x), x_stride, _ptr(weight), None, m, n, k, per_split, splits,
+            _check(self.core.ts_gemm_wide(None, _ptr(out), _ptr(x), x_stride, _ptr(weight), _ptr(bias), m, n, k, per_split, splits,
                                           tile, x_rows, waves, depth, 2, *glu_rule(rule),
                                           self.stream()), "ts_gemm_wide")
             return out
@@ -2253,32 +2355,32 @@ class Ops:
     library_residual_float32 = False
 
     def linear_swiglu(self, x: torch.Tensor, weight: torch.Tensor,
-                      rule: tuple[float, float, float] | None = None) -> torch.Tensor:
+                      rule: tuple[float, float, float] | None = None, bias: torch.Tensor | None = None) -> torch.Tensor:
         """The gated unit of the projection of ``x`` by a gate|up matrix ``[2 I, K]`` whose rows
-        alternate gate, up -> ``[T, I]`` in the dtype of ``x``: ``silu(gate) * up``, or another
+        alternate gate, up (and a bias ``[2 I]`` that alternates likewise) -> ``[T, I]`` in the dtype of ``x``: ``silu(gate) * up``, or another
         unit by ``rule`` (see :meth:`swiglu`).  bfloat16 products that run as one range of K
         apply the unit in the product's own kernel; every other case is the projection followed
         by :meth:`swiglu`."""
         rule = (1.0, 0.0, 0.0) if rule is None else tuple(float(v) for v in rule)
         if x.dtype == torch.bfloat16 and self.skinny_supported(x, weight) and x.shape[0] <= self.skinny_max_rows:
-            _gpu(x, weight)
+            _gpu(x, weight, bias)
             if (self._few_rows_wide(x.shape[0], weight.shape[0], weight.shape[1], 1) and weight.shape[0] % 2 == 0
                     and weight.is_contiguous() and x.stride(1) == 1):
                 wide = self._wide_plan_few_rows(x.shape[0], weight.shape[0], weight.shape[1], 1)
-                return self.gemm_wide(x, weight, plan=wide, gated=True, rule=rule)
+                return self.gemm_wide(x, weight, bias, plan=wide, gated=True, rule=rule)
             plan = self._tiled_plan(x.shape[0], weight.shape[0], weight.shape[1], None)
             if plan[1] == 1 and weight.shape[0] % 2 == 0 and weight.is_contiguous() and x.stride(1) == 1:
-                return self.gemm_tiled(x, weight, plan=plan, gated=True, rule=rule)
+                return self.gemm_tiled(x, weight, bias, plan=plan, gated=True, rule=rule)
         elif (x.dtype == torch.bfloat16 and self.skinny_supported_any_rows(x, weight) and weight.shape[0] % 2 == 0
               and weight.is_contiguous() and x.stride(1) == 1):
-            _gpu(x, weight)
+            _gpu(x, weight, bias)
             m, (n, k) = x.shape[0], weight.shape
             plan = self._wide_plan(m, n, k, True)
-            if self._wide_runs(m, n, k, "gated", plan, lambda: self.gemm_wide(x, weight, plan=plan, gated=True, rule=rule),
-                               lambda: self.swiglu(self._library_product(x, weight, None, None), x.dtype, paired=True, rule=rule)):
-                return self.gemm_wide(x, weight, plan=plan, gated=True, rule=rule)
-            return self.swiglu(self._library_product(x, weight, None, None), x.dtype, paired=True, rule=rule)
-        return self.swiglu(self.linear(x, weight), x.dtype, paired=True, rule=rule)
+            if self._wide_runs(m, n, k, "gated", plan, lambda: self.gemm_wide(x, weight, bias, plan=plan, gated=True, rule=rule),
+                               lambda: self.swiglu(self._library_product(x, weight, bias, None), x.dtype, paired=True, rule=rule)):
+                return self.gemm_wide(x, weight, bias, plan=plan, gated=True, rule=rule)
+            return self.swiglu(self._library_product(x, weight, bias, None), x.dtype, paired=True, rule=rule)
+        return self.swiglu(self.linear(x, weight, bias), x.dtype, paired=True, rule=rule)
 
     def linear(self, x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None = None, *,
                for_residual: bool = False) -> torch.Tensor:

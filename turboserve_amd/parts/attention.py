@@ -278,13 +278,19 @@ class GroupedQueryAttention(Mixer):
         return self.out_size
 
     def scales_its_heads(self) -> bool:
-        """Whether :meth:`heads_out` can apply a scale and write into a wider buffer (the gate's launch does both)."""
-        return self.gate_name is not None
+        """Whether :meth:`heads_out` can apply a scale and write into a wider buffer: the gate's launch does both, and so
+        do the attention kernels that take any rule (the ones that only take plain causal or windowed attention do not)."""
+        return self.gate_name is not None or not self._plain_rule()
+
+    def _plain_rule(self) -> bool:
+        """Whether the head-size-specialised attention kernels take this layer's rule."""
+        return (not self.position.biases_scores and self.value_dim == self.head_dim and self.chunk is None and self.sinks == 0.0
+                and self.keep_first == 0)
 
     def heads_out(self, x: torch.Tensor, ctx, cache, *, scale: float = 1.0, out: tuple | None = None) -> torch.Tensor:
-        """Everything but the output matrix: ``[T, Hq Dv]`` of the run dtype, what that matrix multiplies.  With a gate
-        per head the result may be multiplied by ``scale`` and written into columns of a wider buffer (``out =
-        (buffer, col0)``): a caller that adds this mixer's output to another's can then run both output matrices as
+        """Everything but the output matrix: ``[T, Hq Dv]`` of the run dtype, what that matrix multiplies.  Where
+        :meth:`scales_its_heads` the result may be multiplied by ``scale`` and written into columns of a wider buffer (``out
+        = (buffer, col0)``): a caller that adds this mixer's output to another's can then run both output matrices as
         one product."""
         ops = self.runtime.ops
         qkv = proj = ops.linear(x, self.qkv_weight, self.qkv_bias_tensor)
@@ -323,18 +329,18 @@ class GroupedQueryAttention(Mixer):
         q, q_stride = self.position.encode_and_store(
             qkv, self.num_heads, self.projected_kv_heads, self.head_dim, ctx, cache, **more
         )
+        if self.gate_name is None:
+            return self.attend(q, q_stride, ctx, cache, scale=scale, out=out)
         attended = self.attend(q, q_stride, ctx, cache)
-        if self.gate_name is not None:
-            # Every head's output times the sigmoid of its gate (the projection's last columns), rounded once.
-            return ops.head_gate(attended, proj, self.q_size + self.kv_size + self.v_size, self.num_heads, self.runtime.dtype,
-                                 scale=scale, out=out)
-        if scale != 1.0 or out is not None:
-            raise ValueError(f"{self.prefix}: without a gate per head nothing scales or places the heads' output")
-        return attended
+        # Every head's output times the sigmoid of its gate (the projection's last columns), rounded once.
+        return ops.head_gate(attended, proj, self.q_size + self.kv_size + self.v_size, self.num_heads, self.runtime.dtype,
+                             scale=scale, out=out)
 
-    def attend(self, qkv: torch.Tensor, q_stride: int, ctx, cache: PagedKVView) -> torch.Tensor:
+    def attend(self, qkv: torch.Tensor, q_stride: int, ctx, cache: PagedKVView, *, scale: float = 1.0,
+               out: tuple | None = None) -> torch.Tensor:
         """``[T, Hq D]`` attention output for the step's encoded queries: the first ``Hq D``
-        elements of every ``q_stride``-long row of ``qkv``.
+        elements of every ``q_stride``-long row of ``qkv``; times ``scale``, and into columns of a wider buffer with ``out =
+        (buffer, col0)``, where the layer's rule is not the plain one.
 
         bfloat16 runs use the matrix-core kernels where the geometry allows: one launch for the
         multi-token requests at the front of the batch, one for the single-token requests
@@ -345,9 +351,9 @@ class GroupedQueryAttention(Mixer):
         table = ctx.block_tables[cache.group]
         slopes = self.position.score_slopes(self.num_heads)
         bias = self.position.score_bias_table(self.num_heads)
-        fast = (slopes is None and bias is None and self.value_dim == self.head_dim and self.chunk is None and self.sinks == 0.0
-                and self.keep_first == 0 and ops.mfma_attention_supported(qkv.dtype, self.head_dim, cache.block_size))
-        if fast:
+        if self._plain_rule() and (scale != 1.0 or out is not None):
+            raise ValueError(f"{self.prefix}: plain attention without a gate per head neither scales nor places the heads' output")
+        if self._plain_rule() and ops.mfma_attention_supported(qkv.dtype, self.head_dim, cache.block_size):
             out = ops.rows_buffer(ctx.num_tokens, self.out_size, qkv.dtype, qkv.device)
             if ctx.num_prefill_seqs > 0:
                 # The launch's list of row blocks is the same for every layer with this geometry.
@@ -372,9 +378,9 @@ class GroupedQueryAttention(Mixer):
         if ops.tiled_attention_supported(qkv.dtype, self.head_dim, self.value_dim, cache.block_size, q_stride):
             return tiled_attention(ops, qkv, q_stride, cache.k, cache.v, table, ctx, heads=self.num_heads, scale=self.scale,
                                    window=self.window, chunk=self.chunk, sinks=self.sinks, slopes=slopes, softcap=self.softcap,
-                                   sink_scores=self.sink_scores, distance_bias=bias, keep_first=self.keep_first)
+                                   sink_scores=self.sink_scores, distance_bias=bias, keep_first=self.keep_first, out_scale=scale, out=out)
         return ops.paged_attention_generic(
             qkv, q_stride, cache.k, cache.v, table, ctx.token_seq, ctx.positions,
             self.num_heads, self.scale, self.window, slopes, self.softcap, chunk=self.chunk, sinks=self.sinks,
-            sink_scores=self.sink_scores, distance_bias=bias, keep_first=self.keep_first,
+            sink_scores=self.sink_scores, distance_bias=bias, keep_first=self.keep_first, out_scale=scale, out=out,
         )

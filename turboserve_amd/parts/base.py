@@ -168,10 +168,10 @@ class ResidualStream:
 @dataclass(frozen=True)
 class PendingLayerNorm:
     """The rule of a pending output that passes a layer norm before it is added: the stream gets ``scale *
-    ((p - mean) / sqrt(variance + eps) * weight + bias)``, in 32-bit."""
+    ((p - mean) / sqrt(variance + eps) * weight + bias)``, in 32-bit (a bias of ``None``: nothing is added)."""
 
     weight: torch.Tensor
-    bias: torch.Tensor
+    bias: torch.Tensor | None
     eps: float
     scale: float
 
@@ -255,6 +255,9 @@ class Norm(Part):
 class PositionEncoding(Part):
     """Encodes positions into the queries and keys of an attention mixer and stores the
     step's keys and values into the cache pages (one pass over the projection output)."""
+
+    #: Whether the encoding acts inside the scores (``score_slopes`` or ``score_bias_table``).
+    biases_scores = False
 
     def encode_and_store(
         self,

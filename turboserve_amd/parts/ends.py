@@ -14,15 +14,16 @@ from turboserve_amd.parts.registry import build_part, register_embedding, regist
 
 @register_embedding("token_table")
 class TokenTable(Embedding):
-    """One row of ``[V, H]`` per token id, into the 32-bit residual stream.  ``weight_name``: the
-    table's name under the part's prefix (empty: the prefix itself)."""
+    """One row of ``[V, H]`` per token id, times ``scale`` (in 32-bit), into the 32-bit residual stream.
+    ``weight_name``: the table's name under the part's prefix (empty: the prefix itself)."""
 
     def __init__(self, prefix: str, runtime: Runtime, *, vocab_size: int, hidden_size: int,
-                 weight_name: str = "weight") -> None:
+                 weight_name: str = "weight", scale: float = 1.0) -> None:
         super().__init__(prefix, runtime)
         self.vocab_size = int(vocab_size)
         self.hidden_size = int(hidden_size)
         self.weight_name = weight_name
+        self.scale = float(scale)
         self.weight: torch.Tensor | None = None
 
     def tensor_specs(self) -> dict[str, TensorSpec]:
@@ -32,7 +33,7 @@ class TokenTable(Embedding):
         self.weight = tensors[self.name(self.weight_name)].contiguous()
 
     def forward(self, token_ids: torch.Tensor, ctx) -> torch.Tensor:
-        return self.runtime.ops.embed(self.weight, token_ids)
+        return self.runtime.ops.embed(self.weight, token_ids, scale=self.scale)
 
 
 def sinusoid_table(capacity: int, width: int, base: float) -> torch.Tensor:
@@ -113,8 +114,8 @@ class NormLinearHead(Head):
     """A norm over the summed stream, then ``[V, H]`` without bias, at the wanted rows only
     (model.py:108, :237-244).  ``tied_to`` names the tensor of another part (the token table)
     that serves as the matrix; the checkpoint's own copy under this part's prefix is then not
-    read (the reference shares one parameter, model.py:139-142).  ``softcap = c``: the scores ``z`` leave as
-    ``c tanh(z / c)``."""
+    read (the reference shares one parameter, model.py:139-142).  ``scale = s``: the scores leave as ``s z``;
+    ``softcap = c``: what then is ``z`` leaves as ``c tanh(z / c)``."""
 
     def __init__(
         self,
@@ -128,9 +129,11 @@ class NormLinearHead(Head):
         tied_to: str | None,
         weight_name: str = "weight",
         softcap: float = 0.0,
+        scale: float = 1.0,
     ) -> None:
         super().__init__(prefix, runtime)
         self.softcap = float(softcap)
+        self.scale = float(scale)
         if self.softcap < 0.0:
             raise ValueError(f"a cap of {self.softcap} on the scores")
         self.own_weight_name = weight_name
@@ -165,8 +168,8 @@ class NormLinearHead(Head):
     def forward(self, stream: ResidualStream, rows: torch.Tensor) -> torch.Tensor:
         hidden = self.norm.forward_residual(stream, rows)
         scores = self.runtime.ops.linear_float32_out(hidden, self.weight)
-        if self.softcap > 0.0:
-            scores = self.runtime.ops.tanh_cap(scores.contiguous(), self.softcap)
+        if self.softcap > 0.0 or self.scale != 1.0:
+            scores = self.runtime.ops.scale_cap(scores.contiguous(), scale=self.scale, cap=self.softcap)
         return scores
 
 

@@ -25,7 +25,8 @@ class RoutedExperts(FeedForward):
     is multiplied by ``sigmoid(v . x)``, one number per token, ``v`` the tensor of that name.
 
     Other routers, each a parameter: ``router_scores = "softmax"`` (``s`` is the softmax over all the
-    router's outputs); ``correction_name`` (a vector ``[outputs]`` under the part's prefix that is
+    router's outputs; normalised, the weights are then the softmax over the taken ones alone); ``router_bias_name`` (a
+    vector ``[outputs]`` under the part's prefix that is added, in 32-bit, to what the router's matrix makes); ``correction_name`` (a vector ``[outputs]`` under the part's prefix that is
     added to ``s`` where experts are chosen, while the weights use ``s`` alone); ``normalise =
     False`` (weights ``s * route_scale``, not divided by their sum); ``identity = n`` (the router
     has ``experts + n`` outputs, and the last ``n`` stand for the token itself: such a pair
@@ -62,6 +63,7 @@ class RoutedExperts(FeedForward):
         normalise: bool = True,
         identity: int = 0,
         group_mark: str = "top2_sum",
+        router_bias_name: str | None = None,
     ) -> None:
         super().__init__(prefix, runtime)
         self.hidden_size = int(hidden_size)
@@ -94,6 +96,8 @@ class RoutedExperts(FeedForward):
         self.correction_name = correction_name or None
         self.normalise = bool(normalise)
         self.correction: torch.Tensor | None = None
+        self.router_bias_name = router_bias_name or None
+        self.router_bias: torch.Tensor | None = None  # [outputs] 32-bit
         self.router_name = router_name
         self.expert_names = tuple(expert_names)
         self.shared = None if shared is None else build_part("feed_forward", shared, self.name(shared_name), runtime)
@@ -112,6 +116,8 @@ class RoutedExperts(FeedForward):
         specs = {self.name(self.router_name): TensorSpec((self.outputs, self.hidden_size))}
         if self.correction_name:
             specs[self.name(self.correction_name)] = TensorSpec((self.outputs,), init="zeros")
+        if self.router_bias_name:
+            specs[self.name(self.router_bias_name)] = TensorSpec((self.outputs,), kind="float_keep32", init="zeros")
         for index in range(self.experts):
             specs[self._expert(index, 1)] = TensorSpec((self.expert_size, self.hidden_size))
             specs[self._expert(index, 2)] = TensorSpec((self.expert_size, self.hidden_size))
@@ -133,6 +139,8 @@ class RoutedExperts(FeedForward):
         self.router = tensors[self.name(self.router_name)].contiguous()
         if self.correction_name:
             self.correction = tensors[self.name(self.correction_name)].to(torch.float32).contiguous()
+        if self.router_bias_name:
+            self.router_bias = tensors[self.name(self.router_bias_name)].to(torch.float32).contiguous()
         if self.shared_gate_name:
             # The shared expert's gate is one more row of the router's matrix: one product for both.
             self.router = torch.cat([self.router, tensors[self.shared_gate_name].reshape(1, -1)], dim=0).contiguous()
@@ -151,7 +159,8 @@ class RoutedExperts(FeedForward):
         ops = self.runtime.ops
         taken, weights, gate = ops.moe_route(x, self.router, top=self.top, groups=self.groups, keep=self.keep,
                                              scale=self.route_scale, experts=self.outputs, softmax=self.softmax,
-                                             correction=self.correction, normalise=self.normalise, mark_top=self.mark_top)
+                                             correction=self.correction, normalise=self.normalise, mark_top=self.mark_top,
+                                             bias=self.router_bias)
         grouping = ops.moe_grouping(taken, self.experts, x.dtype, self.hidden_size, self.expert_size)
         units = ops.moe_expert_units(x, self.gate_up, taken, self.rule, grouping)
         outputs = ops.moe_expert_outputs(units, self.down, taken, grouping)

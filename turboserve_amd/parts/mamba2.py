@@ -111,18 +111,8 @@ class Mamba2(Mixer):
         proj = ops.linear(x, self.in_weight)
         u = ops.short_conv(proj, self.inner, self.conv_weight, held.state, ctx.state_slots, ctx.token_seq, ctx.query_start_loc,
                            tokens=ctx.num_tokens, num_seqs=ctx.num_seqs, dtype=dtype, silu=True, bias=self.conv_bias)
-        plan = None
-        if (not ctx.recorded and ctx.max_query_len > ops.selective_walk_tokens
-                and ops.selective_pieces_supported(dtype, self.state_dim, self.value_dim)):
-            # The requests that bring several tokens (they come first) in pieces side by side.
-            piece = ops.selective_piece
-            plan = ctx.derive(("selective_pieces", piece), lambda step: self._plan(step, piece))
+        plan = ops.decaying_plan(ctx, dtype, self.state_dim, self.value_dim)
         y = ops.selective_state(u, proj, self.inner + self.channels, self.dt_bias, self.a_log, self.skip, memory.state, ctx.state_slots,
                                 ctx.query_start_loc, num_seqs=ctx.num_seqs, heads=self.num_heads, groups=self.groups,
                                 state_dim=self.state_dim, value_dim=self.value_dim, dtype=dtype, plan=plan)
         return ops.gated_group_norm(y, proj, 0, self.gain, self.norm_eps, self.norm_groups, dtype)
-
-    def _plan(self, step, piece: int) -> tuple:
-        pieces, carries = self.runtime.ops.linear_state_pieces(step.query_lens[: step.num_prefill_seqs], piece)
-        both = self.runtime.ops.device_ints(pieces + carries)
-        return both[: len(pieces)], both[len(pieces):], len(pieces), len(carries)

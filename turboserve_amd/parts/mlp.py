@@ -21,25 +21,33 @@ class SwiGLU(FeedForward):
     limit)`` and ``u = clamp(up(x), -limit, limit)`` where ``limit > 0``, ``down(g * sigmoid(steepness
     * g) * (u + up_shift))``; the default ``(1, 0, 0)`` is SwiGLU.  A fourth number ``cubic`` makes the
     gate ``g * sigmoid(steepness * (g + cubic * g^3))``; ``ops.GELU_TANH_RULE`` is the tanh form of GELU
-    on the gate.  ``names``: the three matrices' tensor names under the part's prefix."""
+    on the gate.  ``bias``: the three projections have biases, ``<matrix name>.b``.  ``names``: the three matrices' tensor
+    names under the part's prefix."""
 
     def __init__(self, prefix: str, runtime: Runtime, *, hidden_size: int, intermediate_size: int,
                  rule: tuple[float, float, float] = (1.0, 0.0, 0.0),
-                 names: tuple[str, str, str] = ("gate_proj.weight", "up_proj.weight", "down_proj.weight")) -> None:
+                 names: tuple[str, str, str] = ("gate_proj.weight", "up_proj.weight", "down_proj.weight"), bias: bool = False) -> None:
         super().__init__(prefix, runtime)
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.rule = tuple(float(v) for v in rule)
         self.gate_name, self.up_name, self.down_name = names
+        self.bias = bool(bias)
         self.gate_up_weight: torch.Tensor | None = None
+        self.gate_up_bias: torch.Tensor | None = None  # [2 I], alternating like the rows
         self.down_weight: torch.Tensor | None = None
+        self.down_bias: torch.Tensor | None = None
 
     def tensor_specs(self) -> dict[str, TensorSpec]:
-        return {
-            self.name(self.gate_name): TensorSpec((self.intermediate_size, self.hidden_size)),
-            self.name(self.up_name): TensorSpec((self.intermediate_size, self.hidden_size)),
-            self.name(self.down_name): TensorSpec((self.hidden_size, self.intermediate_size)),
+        shapes = {
+            self.gate_name: (self.intermediate_size, self.hidden_size),
+            self.up_name: (self.intermediate_size, self.hidden_size),
+            self.down_name: (self.hidden_size, self.intermediate_size),
         }
+        specs = {self.name(name): TensorSpec(shape) for name, shape in shapes.items()}
+        if self.bias:
+            specs.update({self.name(f"{name}.b"): TensorSpec(shape[:1], init="zeros") for name, shape in shapes.items()})
+        return specs
 
     def activation_bytes(self, tokens: int, itemsize: int) -> int:
         """The gate|up projection, the activated product and the down projection (32-bit: it is
@@ -50,10 +58,14 @@ class SwiGLU(FeedForward):
         gate, up = tensors[self.name(self.gate_name)], tensors[self.name(self.up_name)]
         self.gate_up_weight = torch.stack([gate, up], dim=1).reshape(2 * gate.shape[0], gate.shape[1]).contiguous()
         self.down_weight = tensors[self.name(self.down_name)].contiguous()
+        if self.bias:
+            gate, up, self.down_bias = (tensors[self.name(f"{n}.b")].contiguous() for n in (self.gate_name, self.up_name, self.down_name))
+            self.gate_up_bias = torch.stack([gate, up], dim=1).reshape(-1).contiguous()
 
     def forward(self, x: torch.Tensor, ctx) -> torch.Tensor:
         ops = self.runtime.ops
-        return ops.linear(ops.linear_swiglu(x, self.gate_up_weight, self.rule), self.down_weight, for_residual=True)
+        units = ops.linear_swiglu(x, self.gate_up_weight, self.rule, self.gate_up_bias)
+        return ops.linear(units, self.down_weight, self.down_bias, for_residual=True)
 
 
 @register_feed_forward("mlp")

@@ -129,10 +129,11 @@ def _layer_normed_pending(norm: Norm, stream: ResidualStream, rows: torch.Tensor
 class LayerNorm(Norm):
     """``(x - mean) / sqrt(variance + eps) * weight + bias``, the variance being the mean of the squared deviations, in
     32-bit with one rounding.  The fused form also carries the residual sum, kept in 32-bit.  ``weight_name``: the
-    weight's name under the part's prefix (empty: the prefix itself); ``bias_name`` is appended to the weight's name."""
+    weight's name under the part's prefix (empty: the prefix itself); ``bias_name`` is appended to the weight's name
+    (``None``: the norm has no bias)."""
 
     def __init__(self, prefix: str, runtime: Runtime, *, size: int, eps: float, weight_name: str = "weight",
-                 bias_name: str = "b") -> None:
+                 bias_name: str | None = "b") -> None:
         super().__init__(prefix, runtime)
         self.size = int(size)
         self.eps = float(eps)
@@ -146,14 +147,18 @@ class LayerNorm(Norm):
         return f"{self.name(self.weight_name)}.{self.bias_name}"
 
     def tensor_specs(self) -> dict[str, TensorSpec]:
-        return {self.name(self.weight_name): TensorSpec((self.size,), init="ones"), self._bias(): TensorSpec((self.size,), init="zeros")}
+        specs = {self.name(self.weight_name): TensorSpec((self.size,), init="ones")}
+        if self.bias_name is not None:
+            specs[self._bias()] = TensorSpec((self.size,), init="zeros")
+        return specs
 
     def activation_bytes(self, tokens: int, itemsize: int) -> int:
         return tokens * self.size * itemsize
 
     def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
         self.weight = tensors[self.name(self.weight_name)].contiguous()
-        self.bias = tensors[self._bias()].contiguous()
+        if self.bias_name is not None:
+            self.bias = tensors[self._bias()].contiguous()
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError(f"{self.prefix}: this norm runs where it carries the residual sum")

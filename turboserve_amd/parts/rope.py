@@ -230,6 +230,7 @@ class DistanceSlopes(NoPositionEncoding):
     projected."""
 
     shareable = True
+    biases_scores = True
 
     def __init__(self, prefix: str, runtime: Runtime, *, exponent: float = 8.0) -> None:
         super().__init__(prefix, runtime)
@@ -264,6 +265,7 @@ class DistanceBuckets(NoPositionEncoding):
     ``reach``, if that is shorter): the attention kernels read it by ``min(n, L - 1)``."""
 
     shareable = False
+    biases_scores = True
 
     def __init__(self, prefix: str, runtime: Runtime, *, num_heads: int, max_distance: float, buckets: int | None = None,
                  reach: int | None = None, table_name: str = "rel") -> None:
