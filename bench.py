@@ -33,7 +33,7 @@ and one 2,048-token prompt), ``--shape 32b --batch 64 --fill-hbm`` (a cache pool
 free memory), ``--closed-loop C [--sampled]`` (the reference's serving profile driven offline: 256
 requests of 128..1,024 tokens in and 64..512 out, C in flight; the library's products run at a
 few step sizes that are all timed at start-up, about 70 s the first time), ``--attention-prefill T[,CTX]`` (the
-prefill attention kernel alone), ``--sample-kernel ROWS`` (the sampling kernel alone), ``--hbm-read`` (a kernel that only reads: what the memory gives), ``--only-prefill [TOKENS]`` (one prompt's prefill alone, 2,048 tokens or TOKENS), ``--designs [2k,4k]`` (the Sisisun design beside a Qwen2 model of equal layer sizes: prefill and decode; with ``--design kisadra`` the Kisadra design beside Sisisun, with ``--design dovudra`` the Dovudra design beside Kisadra, with ``--design legavik`` the Legavik design beside Kisadra, with ``--design lukelix`` the Lukelix design beside Kisadra), ``--kernel-shares TRACE.csv`` (no GPU: the per-kernel table of a
+prefill attention kernel alone), ``--sample-kernel ROWS`` (the sampling kernel alone), ``--hbm-read`` (a kernel that only reads: what the memory gives), ``--only-prefill [TOKENS]`` (one prompt's prefill alone, 2,048 tokens or TOKENS), ``--designs [2k,4k]`` (the Sisisun design beside a Qwen2 model of equal layer sizes: prefill and decode; with ``--design kisadra`` the Kisadra design beside Sisisun, with ``--design dovudra`` the Dovudra design beside Kisadra, with ``--design legavik`` the Legavik design beside Kisadra, with ``--design lukelix`` the Lukelix design beside Kisadra, with ``--design ninenex`` the Ninenex design beside Kisadra), ``--kernel-shares TRACE.csv`` (no GPU: the per-kernel table of a
 ``rocprofv3 --kernel-trace`` of any of these runs).
 """
 
@@ -124,9 +124,9 @@ def parse_args(argv: list[str] | None = None) -> argparse.Namespace:
                    help="prefill and decode of the Sisisun design (random weights) at layer sizes that resemble a real "
                         "model's (2k, 4k: the width), beside a Qwen2 model of the same width, heads, feed-forward and "
                         "number of layer runs; prints one JSON object and exits")
-    p.add_argument("--design", choices=["sisisun", "kisadra", "dovudra", "legavik", "lukelix"], default="sisisun",
+    p.add_argument("--design", choices=["sisisun", "kisadra", "dovudra", "legavik", "lukelix", "ninenex"], default="sisisun",
                    help="which design --designs measures: sisisun beside Qwen2, kisadra beside sisisun, dovudra beside kisadra, "
-                        "legavik beside kisadra, or lukelix beside kisadra")
+                        "legavik beside kisadra, lukelix beside kisadra, or ninenex beside kisadra")
     return p.parse_args(argv)
 
 
@@ -602,6 +602,41 @@ def lukelix_pair(size: str) -> tuple[dict, dict]:
     return lukelix, kisadra
 
 
+#: ``--designs --design ninenex``: the Ninenex configuration of a size (eight layers, a matrix memory and a pair of chunked
+#: attention and retention in turn, dense and routed feed-forwards in turn) beside a Kisadra configuration of the same
+#: mixers' sizes: gated linear attention in the matrix memory's heads for every such layer; for every pair an attention layer
+#: with the same chunks and without a feed-forward, and a gated-linear-attention layer in the retention's heads with the
+#: pair's feed-forward; the same dense feed-forwards and experts (the shared expert as one more routed one).
+def ninenex_pair(size: str) -> tuple[dict, dict]:
+    width, heads, kv, ff, experts, top, expert_ff = {"2k": (2048, 16, 4, 8192, 32, 4, 1024), "4k": (4096, 32, 8, 14336, 64, 6, 1408)}[size]
+    chunk = {"size": 8192}
+    memory = {"heads": width // 512, "dim": 256, "vdim": 512}  # keys half as wide as the model, values as wide
+    attention = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": chunk}
+    kept = {"heads": width // 256, "dim": 128, "vdim": 256}
+    pair = {"left": dict(attention, rot={"base": 500000.0, "dims": 64}),
+            "right": dict(kept, decay=[1.0 - 2.0 ** (-5 - 7.0 * h / kept["heads"]) for h in range(kept["heads"])]),
+            "left_scale": 0.7, "right_scale": 0.7}
+    dense = {"kind": "dense", "ff": ff}
+    routed = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": expert_ff}}
+    beside_routed = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "router": {"experts": experts + 1, "top": top + 1}}
+    layers, beside = [], []
+    for index in range(8):
+        is_dense = index % 4 in (0, 3)
+        mlp, other = dense if is_dense else routed, dense if is_dense else beside_routed
+        if index % 2 == 0:
+            layers.append({"type": "mlstm", "mixer": dict(memory, gate_cap=15.0), "mlp": mlp})
+            beside.append({"type": "gla", "mixer": dict(memory, tau=16.0, rank=16), "mlp": other})
+        else:
+            layers.append({"type": "parallel", "mixer": pair, "mlp": mlp})
+            beside.append({"type": "attention", "mixer": attention, "mlp": None})
+            beside.append({"type": "gla", "mixer": dict(kept, tau=16.0, rank=16), "mlp": other})
+    ninenex = {"architecture": "Ninenex", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 3.0},
+               "logit_scale": 0.25, "layers": layers}
+    kisadra = {"architecture": "Kisadra", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "layers": beside,
+               "loop": {"start": 0, "stop": 0, "times": 1}}
+    return ninenex, kisadra
+
+
 def mixer_work(mixer, batch: int, context: int, prompt: int) -> tuple[float, float]:
     """``(elements a decode step of `batch` requests at `context` tokens reads from the cache or state,
     multiply-adds x 2 of a prompt of `prompt` tokens inside the mixer beside its plain projections)``."""
@@ -617,6 +652,9 @@ def mixer_work(mixer, batch: int, context: int, prompt: int) -> tuple[float, flo
     if kind == "Mamba2":
         state = mixer.num_heads * mixer.state_dim * mixer.value_dim
         return batch * (2 * state * 2.0 + 4.0 * (mixer.taps - 1) * mixer.channels), 4.0 * prompt * state
+    if kind in ("MatrixMemory", "Retention"):
+        state = mixer.num_heads * mixer.head_dim * (mixer.value_dim + (1 if kind == "MatrixMemory" else 0))
+        return batch * 2 * state * 2.0, 4.0 * prompt * state
     if kind == "GatedLinearAttention":
         state = mixer.num_heads * mixer.head_dim * mixer.value_dim
         return batch * 2 * state * 2.0, 4.0 * prompt * state  # 32-bit state read and written: 2 x 2 run-dtype elements
@@ -671,7 +709,7 @@ def run_designs(sizes: list[str], dtype_name: str, steps: int, warmup: int, desi
     for size in sizes:
         size, _, only = size.partition(":")  # "2k:qwen2": that design alone; "2k:qwen2:prefill": that phase alone (for profiles)
         only, _, phase = only.partition(":")
-        labels, pair = {"lukelix": (("lukelix", "kisadra"), lukelix_pair), "legavik": (("legavik", "kisadra"), legavik_pair),
+        labels, pair = {"ninenex": (("ninenex", "kisadra"), ninenex_pair), "lukelix": (("lukelix", "kisadra"), lukelix_pair), "legavik": (("legavik", "kisadra"), legavik_pair),
                         "dovudra": (("dovudra", "kisadra"), dovudra_pair), "kisadra": (("kisadra", "sisisun"), kisadra_pair),
                         "sisisun": (("sisisun", "qwen2"), lambda s: design_pair(s))}[design]
         pair = pair(size)

@@ -47,6 +47,11 @@ def capped_gates(i_raw: torch.Tensor, f_raw: torch.Tensor, cap: float) -> tuple[
     return cap * torch.tanh(i_raw / cap), torch.nn.functional.logsigmoid(cap * torch.tanh(f_raw / cap))
 
 
+def least(m: torch.Tensor) -> torch.Tensor:
+    """What a read-out is divided by at least."""
+    return torch.exp(-m)
+
+
 def memory_walk(q, k, v, i, f) -> torch.Tensor:
     """One head: ``q, k [T, D]`` (``q`` scaled), ``v [T, Dv]``, log gates ``i, f [T]`` -> ``[T, Dv]``."""
     S = torch.zeros(q.shape[1], v.shape[1], dtype=q.dtype)
@@ -59,7 +64,7 @@ def memory_walk(q, k, v, i, f) -> torch.Tensor:
         m = top
         S = keep * S + add * torch.outer(k[t], v[t])
         n = keep * n + add * k[t]
-        out[t] = (S.T @ q[t]) / (torch.maximum((n @ q[t]).abs(), torch.exp(-m)) + 1e-6)
+        out[t] = (S.T @ q[t]) / (torch.maximum((n @ q[t]).abs(), least(m)) + 1e-6)
     return out
 
 

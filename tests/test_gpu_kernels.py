@@ -211,9 +211,13 @@ def test_gemm_tiled_applies_swiglu_itself(ops, tile, m, inter, k):
     exact = ops.linear_swiglu(x.float().to(DEV), w.float().to(DEV))
     assert exact.dtype == torch.float32
     assert float((exact.double().cpu() - want).abs().max()) <= 1e-5 * float(want.abs().max() + 1) * math.sqrt(k)
-    with pytest.raises(Exception, match="one range of K"):
-        ops.gemm_tiled(x.to(DEV), w.to(DEV), plan=(1, -(-k // 128), tile), gated=True) if k > 128 else ops.gemm_tiled(
-            x.to(DEV), w.to(DEV), torch.zeros(2 * inter).bfloat16().to(DEV), plan=plan, gated=True)
+    # A bias that alternates like the rows is added before the unit.
+    bias = torch.randn(2 * inter, generator=g).bfloat16().to(DEV)
+    fused = ops.gemm_tiled(x.to(DEV), w.to(DEV), bias, plan=plan, gated=True)
+    assert torch.equal(fused, ops.swiglu(ops.gemm_tiled(x.to(DEV), w.to(DEV), bias, plan=plan), torch.bfloat16, paired=True))
+    if k > 128:
+        with pytest.raises(Exception, match="one range of K"):
+            ops.gemm_tiled(x.to(DEV), w.to(DEV), plan=(1, -(-k // 128), tile), gated=True)
 
 
 WIDE_GRIDS = [(2, 128, 4), (4, 128, 4), (5, 128, 4), (2, 256, 4), (4, 256, 4), (5, 256, 4),
@@ -254,9 +258,13 @@ def test_gemm_wide_every_tile_and_grid(ops, tile, x_rows, waves, m, n, k):
         assert float((fused.double().cpu() - gated).abs().max()) <= 1e-2 * float(gated.abs().max() + 1)
         # the fused form rounds once, the two-kernel form twice: equal up to that
         assert float((fused.double() - two_steps.double()).abs().max()) <= 1e-2 * float(gated.abs().max() + 1)
-    with pytest.raises(Exception, match="one range of K"):
-        ops.gemm_wide(x.to(DEV), w.to(DEV), plan=(1, iters, tile, x_rows, waves), gated=True) if iters > 1 else ops.gemm_wide(
-            x.to(DEV), w.to(DEV), b.to(DEV), plan=(iters, 1, tile, x_rows, waves), gated=True)
+        # a bias that alternates like the rows is added before the unit
+        biased = ops.gemm_wide(x.to(DEV), w.to(DEV), b.to(DEV), plan=(iters, 1, tile, x_rows, waves), gated=True)
+        gated = torch.nn.functional.silu(want[:, 0::2]) * want[:, 1::2]
+        assert float((biased.double().cpu() - gated).abs().max()) <= 1e-2 * float(gated.abs().max() + 1)
+    if n % 2 == 1 or iters > 1:
+        with pytest.raises(Exception, match="one range of K"):
+            ops.gemm_wide(x.to(DEV), w.to(DEV), plan=(1, iters, tile, x_rows, waves), gated=True)
 
 
 @pytest.mark.parametrize("tile,x_rows,depth", [(2, 64, 64), (4, 64, 64), (5, 64, 64), (8, 64, 64), (2, 64, 128), (4, 64, 128),

@@ -353,7 +353,7 @@ class GroupedQueryAttention(Mixer):
         bias = self.position.score_bias_table(self.num_heads)
         if self._plain_rule() and (scale != 1.0 or out is not None):
             raise ValueError(f"{self.prefix}: plain attention without a gate per head neither scales nor places the heads' output")
-        if self._plain_rule() and ops.mfma_attention_supported(qkv.dtype, self.head_dim, cache.block_size):
+        if self._plain_rule() and slopes is None and bias is None and ops.mfma_attention_supported(qkv.dtype, self.head_dim, cache.block_size):
             out = ops.rows_buffer(ctx.num_tokens, self.out_size, qkv.dtype, qkv.device)
             if ctx.num_prefill_seqs > 0:
                 # The launch's list of row blocks is the same for every layer with this geometry.
