@@ -65,6 +65,31 @@ __device__ __forceinline__ float ss_input(const P* p, int splits, size_t stride)
   return s;
 }
 
+// Two at once, twice as many loads in flight.
+template <typename P>
+__device__ __forceinline__ void ss_input_two(const P* p, const P* q, int splits, size_t stride, float& a, float& b) {
+  if (splits == 1) {
+    a = to_float(p[0]);
+    b = to_float(q[0]);
+    return;
+  }
+  a = b = 0.f;
+  for (int first = 0; first < splits; first += 8) {
+    float v[8], w[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      v[j] = to_float(p[(size_t)min(first + j, splits - 1) * stride]);
+      w[j] = to_float(q[(size_t)min(first + j, splits - 1) * stride]);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (first + j < splits) {
+        a += v[j];
+        b += w[j];
+      }
+  }
+}
+
 // The same of VEC neighbouring elements.
 template <typename P, int VEC>
 __device__ __forceinline__ void ss_input_vec(const P* p, int splits, size_t stride, float (&v)[VEC]) {
@@ -113,8 +138,10 @@ __device__ __forceinline__ float ss_log_sigmoid(float z) { return fminf(z, 0.f) 
 template <typename P>
 __device__ __forceinline__ void ss_log_gates(const P* proj, const SsGates& gates, int t, int h, int heads, float& in, float& forget) {
   const P* row = proj + (size_t)t * gates.width + gates.first + h;
-  in = ss_capped(ss_input(row, gates.splits, gates.stride) + gates.one[h], gates.cap);
-  forget = ss_log_sigmoid(ss_capped(ss_input(row + heads, gates.splits, gates.stride) + gates.two[h], gates.cap));
+  float i, f;
+  ss_input_two(row, row + heads, gates.splits, gates.stride, i, f);
+  in = ss_capped(i + gates.one[h], gates.cap);
+  forget = ss_log_sigmoid(ss_capped(f + gates.two[h], gates.cap));
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -124,7 +151,7 @@ __device__ __forceinline__ void ss_log_gates(const P* proj, const SsGates& gates
 // NR: state rows a thread holds (of every stretch of 4 SS_PARTS rows the four from 4 part on); COLS: columns of a
 // workgroup; BATCH: tokens staged in LDS at a time.  norm [T, H, 2] (gated): n . C and the running maximum.
 template <typename U, typename P, int RULE, int NR, int BATCH, int COLS>
-__global__ void __launch_bounds__(SS_PARTS * COLS)
+__global__ void __launch_bounds__(SS_PARTS * COLS, NR <= 32 ? 5 : 2)
 decaying_walk_kernel(float* __restrict__ y, float* __restrict__ norm, float* __restrict__ state, float* __restrict__ sums,
                      const float* __restrict__ tops, const U* __restrict__ u, SsRows rows, const P* __restrict__ proj, SsGates gates,
                      const float* __restrict__ skip, float scale, const int* __restrict__ state_slots,
@@ -170,39 +197,43 @@ decaying_walk_kernel(float* __restrict__ y, float* __restrict__ norm, float* __r
   for (int base = 0; base < count; base += BATCH) {
     const int batch = min(BATCH, count - base);
     if (base > 0) __syncthreads();  // the batch before is done with what is staged
-    for (int i = tid; i < batch * ROWS; i += THREADS) {
-      const int j = i / ROWS, d = i % ROWS;
-      const U* row = u + (size_t)(row0 + base + j) * rows.width;
-      bs[j][d] = d < n ? ss_input(row + b_at + d, rows.splits, rows.stride) : 0.f;
-      cs[j][d] = d < n ? ss_input(row + c_at + d, rows.splits, rows.stride) : 0.f;
+    // The gates are the second wavefront's, x the last ones': a step of one token waits for them side by side.
+    const int lane = tid - TS_WAVE;
+    if (RULE == SS_SELECTIVE && lane >= 0 && lane < batch) {
+      const float dt = ss_softplus(ss_input(proj + (size_t)(row0 + base + lane) * gates.width + gates.first + h, gates.splits, gates.stride) + bias);
+      ws[lane] = dt;
+      as[lane] = expf(-rate * dt);
     }
-    for (int i = tid; i < batch * COLS; i += THREADS) {
-      const int j = i / COLS, cc = c0 + i % COLS;
-      float v = RULE == SS_GATED && cc == p ? 1.f : 0.f;
-      if (cc < p) v = ss_input(u + (size_t)(row0 + base + j) * rows.width + x_at + cc, rows.splits, rows.stride);
-      xs[j][i % COLS] = v;
+    if (RULE == SS_FIXED && lane >= 0 && lane < batch) {
+      ws[lane] = 1.f;
+      as[lane] = rate;
     }
-    if (RULE == SS_SELECTIVE && tid < batch) {
-      const float dt = ss_softplus(ss_input(proj + (size_t)(row0 + base + tid) * gates.width + gates.first + h, gates.splits, gates.stride) + bias);
-      ws[tid] = dt;
-      as[tid] = expf(-rate * dt);
-    }
-    if (RULE == SS_FIXED && tid < batch) {
-      ws[tid] = 1.f;
-      as[tid] = rate;
-    }
-    if (RULE == SS_GATED && tid < TS_WAVE) {  // lane j takes token j's gates; the maximum passes from token to token
+    if (RULE == SS_GATED && lane >= 0 && lane < TS_WAVE) {  // lane j takes token j's gates; the maximum passes from token to token
       float in, forget;
-      ss_log_gates(proj, gates, row0 + base + min(tid, batch - 1), h, heads, in, forget);
+      ss_log_gates(proj, gates, row0 + base + min(lane, batch - 1), h, heads, in, forget);
       for (int j = 0; j < batch; ++j) {
         const float i = __shfl(in, j), f = __shfl(forget, j), next = fmaxf(f + top, i);
-        if (tid == j) {
+        if (lane == j) {
           ws[j] = expf(i - next);
           as[j] = expf(f + top - next);
           ms[j] = next;
         }
         top = next;
       }
+    }
+    for (int i = THREADS - 1 - tid; i < batch * COLS; i += THREADS) {
+      const int j = i / COLS, cc = c0 + i % COLS;
+      float v = RULE == SS_GATED && cc == p ? 1.f : 0.f;
+      if (cc < p) v = ss_input(u + (size_t)(row0 + base + j) * rows.width + x_at + cc, rows.splits, rows.stride);
+      xs[j][i % COLS] = v;
+    }
+    for (int i = tid; i < batch * ROWS; i += THREADS) {
+      const int j = i / ROWS, d = i % ROWS;
+      const U* row = u + (size_t)(row0 + base + j) * rows.width;
+      float vb = 0.f, vc = 0.f;
+      if (d < n) ss_input_two(row + b_at + d, row + c_at + d, rows.splits, rows.stride, vb, vc);
+      bs[j][d] = vb;
+      cs[j][d] = vc;
     }
     __syncthreads();
     for (int j = 0; j < batch; ++j) {
@@ -875,29 +906,49 @@ heads_finish_kernel(T* __restrict__ out, size_t out_stride, const float* __restr
     if (lane == 0 && t + 1 == query_start_loc[seq + 1]) tops[(size_t)state_slots[seq] * heads + h] = m;
   }
   const float* row = y + (size_t)item * p;
-  float ss = 0.f;
-  for (int i = lane * VEC; i < p; i += TS_WAVE * VEC) {
-    float v[VEC];
-    load_vec<float, VEC>(row + i, v);
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) ss = fmaf(v[e] * inv, v[e] * inv, ss);
-  }
-  const float by = inv * rsqrtf(wave_sum(ss) / (float)p + eps) * scale;
   const P* gates = proj + (size_t)t * width + gate_at + (size_t)h * p;
   T* to = out + (size_t)t * out_stride + (size_t)h * p;
-  for (int i = lane * VEC; i < p; i += TS_WAVE * VEC) {
-    float v[VEC], z[VEC];
-    ss_input_vec<P, VEC>(gates + i, splits, split_stride, z);
-    load_vec<float, VEC>(row + i, v);
+  // A wavefront's first HELD turns stay in registers, the gates asked for before the sum is waited for.
+  constexpr int HELD = 2;
+  float v[HELD][VEC], z[HELD][VEC];
+  float ss = 0.f;
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) v[e] *= by * ((sigmoid ? 1.f : z[e]) / (1.f + expf(-z[e])));
+  for (int c = 0; c < HELD; ++c) {
+    const int i = (c * TS_WAVE + lane) * VEC;
+    if (i >= p) continue;
+    load_vec<float, VEC>(row + i, v[c]);
+    ss_input_vec<P, VEC>(gates + i, splits, split_stride, z[c]);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss = fmaf(v[c][e] * inv, v[c][e] * inv, ss);
+  }
+  for (int i = (HELD * TS_WAVE + lane) * VEC; i < p; i += TS_WAVE * VEC) {
+    float more[VEC];
+    load_vec<float, VEC>(row + i, more);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss = fmaf(more[e] * inv, more[e] * inv, ss);
+  }
+  const float by = inv * rsqrtf(wave_sum(ss) / (float)p + eps) * scale;
+  auto leave = [&](int i, float (&value)[VEC], const float (&gate)[VEC]) __attribute__((always_inline)) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) value[e] *= by * ((sigmoid ? 1.f : gate[e]) / (1.f + expf(-gate[e])));
     if (gain) {
       float w[VEC];
       load_vec<T, VEC>(gain + (size_t)h * p + i, w);
 #pragma unroll
-      for (int e = 0; e < VEC; ++e) v[e] *= w[e];
+      for (int e = 0; e < VEC; ++e) value[e] *= w[e];
     }
-    store_vec<T, VEC>(to + i, v);
+    store_vec<T, VEC>(to + i, value);
+  };
+#pragma unroll
+  for (int c = 0; c < HELD; ++c) {
+    const int i = (c * TS_WAVE + lane) * VEC;
+    if (i < p) leave(i, v[c], z[c]);
+  }
+  for (int i = (HELD * TS_WAVE + lane) * VEC; i < p; i += TS_WAVE * VEC) {
+    float more[VEC], gate[VEC];
+    load_vec<float, VEC>(row + i, more);
+    ss_input_vec<P, VEC>(gates + i, splits, split_stride, gate);
+    leave(i, more, gate);
   }
 }
 
