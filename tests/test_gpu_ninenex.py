@@ -349,6 +349,39 @@ def test_the_router_with_a_bias(ops, dtype, experts, top):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("normed", [False, True])
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,turned,tokens", [
+    (4, 2, 16, 24, 16, 40), (3, 3, 12, 12, 8, 45), (2, 1, 128, 128, 128, 70), (8, 1, 128, 64, 64, 35), (1, 1, 64, 80, 48, 33), (6, 2, 72, 40, 32, 90),
+    (2, 2, 40, 40, 12, 37), (3, 1, 96, 96, 96, 5)])
+def test_the_store_turns_halves_of_a_heads_first_elements(ops, dtype, normed, heads, kv_heads, dim, vdim, turned, tokens):
+    """In prompts (also where a pair lies in two lanes) and in steps of few tokens, with a norm per head and without."""
+    g = torch.Generator().manual_seed(dim + tokens)
+    page, first = 8, 29
+    proj = torch.randn(tokens, (heads + kv_heads) * dim + kv_heads * vdim, generator=g).to(dtype)
+    gains = [(1 + 0.3 * torch.randn(dim, generator=g)).to(dtype) for _ in range(2)]
+    rot = {"base": 70.0, "dims": turned}
+    angles = torch.outer(torch.arange(first + tokens, dtype=torch.float64), 70.0 ** (-2.0 * torch.arange(turned // 2, dtype=torch.float64) / turned))
+    padded = torch.cat([torch.zeros(first, proj.shape[1]), proj.float()])
+
+    def turn(columns, count, gain):
+        x = padded[:, columns:columns + count * dim].view(-1, count, dim)
+        return plain.turn_halves(plain.unit_rms(x, 1e-5) * gain.float() if normed else x, rot)[first:]
+
+    pages = -(-(first + tokens) // page)
+    order = torch.randperm(pages, generator=g)
+    slots = torch.tensor([int(order[p // page]) * page + p % page for p in range(first, first + tokens)])
+    k_pages = torch.zeros(pages, kv_heads, page, dim, dtype=dtype, device=DEV)
+    v_pages = torch.zeros(pages, kv_heads, vdim, page, dtype=dtype, device=DEV)
+    q, stride = ops.head_norm_store(
+        proj.clone().to(DEV), k_pages, v_pages, *(gain.to(DEV) if normed else None for gain in gains), 1e-5, ints(range(first, first + tokens)),
+        slots.to(torch.int32).to(DEV), heads, kv_heads, dim, vdim, page, dtype, cos=angles.cos().float().to(DEV),
+        sin=angles.sin().float().to(DEV), max_position=first + tokens - 1)
+    near(q.view(tokens, -1)[:, :heads * dim], turn(0, heads, gains[0]).reshape(tokens, -1), dtype)
+    near(k_pages[slots // page, :, slots % page], turn(heads * dim, kv_heads, gains[1]), dtype)
+    near(v_pages[slots // page, :, :, slots % page], proj.float()[:, (heads + kv_heads) * dim:].view(tokens, kv_heads, vdim), dtype)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(4, 2, 16, 24), (3, 1, 20, 12), (8, 1, 64, 80)])
 def test_attention_scales_and_places_its_heads(ops, dtype, heads, kv_heads, dim, vdim):
     """A portion and a single token behind it, the keys of the single token shared out over several workgroups: the same

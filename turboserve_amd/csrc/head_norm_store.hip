@@ -171,8 +171,9 @@ head_norm_store_kernel(T* q_out, long q_stride, const P* proj, int splits, size_
   }
 }
 
-// The same for many tokens (prompt portions): bfloat16 in and out, no partial sums, no rotation or one of
-// neighbouring pairs (a multiple of 8 elements of a head), head size a multiple of 8 and at most 128.  Sixteen lanes per (token, q or k head), eight
+// The same for many tokens (prompt portions): bfloat16 in and out, no partial sums, no rotation, one of
+// neighbouring pairs (a multiple of 8 elements of a head) or one in halves (of 16: a pair's two elements then lie in two
+// lanes that hand them to each other), head size a multiple of 8 and at most 128.  Sixteen lanes per (token, q or k head), eight
 // elements a lane with one 16-byte load and one 16-byte store; the sum of squares is formed over
 // the sixteen lanes of a row by data-parallel moves.  Per element the arithmetic of the kernel
 // above.
@@ -180,8 +181,8 @@ __global__ void __launch_bounds__(256)
 head_norm_store_rows_kernel(bf16_t* q_out, long q_stride, const bf16_t* proj, bf16_t* __restrict__ k_pages,
                             const bf16_t* __restrict__ q_gain, const bf16_t* __restrict__ k_gain, float eps,
                             float gain_offset, const float* __restrict__ cos_table, const float* __restrict__ sin_table,
-                            const int* __restrict__ positions, int turned, const int* __restrict__ slots, int tokens, int heads,
-                            int kv_heads, int dim, int vdim, int block_size) {
+                            const int* __restrict__ positions, int turned, int neighbours, const int* __restrict__ slots, int tokens,
+                            int heads, int kv_heads, int dim, int vdim, int block_size) {
   const int qk_heads = heads + kv_heads;
   const long items = (long)tokens * qk_heads;
   const long asked = (long)blockIdx.x * 16 + threadIdx.x / 16;
@@ -218,7 +219,26 @@ head_norm_store_rows_kernel(bf16_t* q_out, long q_stride, const bf16_t* proj, bf
 #pragma unroll
     for (int e = 0; e < 8; ++e) x[e] = x[e] * r * (gain_offset + g[e]);
   }
-  if (cos_table && piece * 8 < turned) {  // the lane's four pairs
+  if (cos_table && !neighbours) {
+    const int half = turned / 16;  // pieces of a half; piece p < half goes with piece p + half
+    const bool second = piece >= half, in = piece < 2 * half;
+    const int mine = second ? piece - half : piece, partner = !in ? piece : second ? mine : piece + half;
+    float other[8], cs[8], sn[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) other[e] = __shfl(x[e], (threadIdx.x & (TS_WAVE - 16)) + partner);
+    if (in) {
+      const size_t at = (size_t)positions[t] * (turned / 2) + mine * 8;
+#pragma unroll
+      for (int e = 0; e < 8; e += 4) {
+        const float4 cv = *reinterpret_cast<const float4*>(cos_table + at + e), sv = *reinterpret_cast<const float4*>(sin_table + at + e);
+        cs[e] = cv.x; cs[e + 1] = cv.y; cs[e + 2] = cv.z; cs[e + 3] = cv.w;
+        sn[e] = sv.x; sn[e + 1] = sv.y; sn[e + 2] = sv.z; sn[e + 3] = sv.w;
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = second ? __builtin_fmaf(x[e], cs[e], other[e] * sn[e]) : __builtin_fmaf(x[e], cs[e], -(other[e] * sn[e]));
+    }
+  }
+  if (cos_table && neighbours && piece * 8 < turned) {  // the lane's four pairs
     const size_t at = (size_t)positions[t] * (turned / 2) + piece * 4;
     const float4 cv = *reinterpret_cast<const float4*>(cos_table + at), sv = *reinterpret_cast<const float4*>(sin_table + at);
     const float cs[4] = {cv.x, cv.y, cv.z, cv.w}, sn[4] = {sv.x, sv.y, sv.z, sv.w};
@@ -298,12 +318,13 @@ static void launch_head_norm_store(void* q_out, long q_stride, const void* proj,
                        q_stride % 8 == 0 && vdim % 8 == 0;
   const bool plain = (!shape.normed || q_gain) && !shape.norm_after && !shape.values_are_keys && shape.temp_coef == 0.f && shape.tail == 0;
   const int turned = shape.rot_dims > 0 ? shape.rot_dims : dim;
-  const bool in_lanes = !cos_table || (shape.neighbours && turned % 8 == 0 && ((uintptr_t)cos_table | (uintptr_t)sin_table) % 16 == 0);
+  const bool in_lanes = !cos_table || (turned % (shape.neighbours ? 8 : 16) == 0 && ((uintptr_t)cos_table | (uintptr_t)sin_table) % 16 == 0);
   if (std::is_same<T, bf16_t>::value && std::is_same<P, bf16_t>::value && splits == 1 && in_lanes && dim % 8 == 0 &&
       dim <= 128 && !few && aligned && plain)
     hipLaunchKernelGGL(head_norm_store_rows_kernel, dim3((unsigned)((items + 15) / 16)), dim3(256), 0, stream, (bf16_t*)q_out,
                        q_stride, (const bf16_t*)proj, (bf16_t*)k_pages, (const bf16_t*)q_gain, (const bf16_t*)k_gain, eps,
-                       gain_offset, cos_table, sin_table, positions, turned, slots, tokens, heads, kv_heads, dim, vdim, block_size);
+                       gain_offset, cos_table, sin_table, positions, turned, shape.neighbours, slots, tokens, heads, kv_heads, dim, vdim,
+                       block_size);
   else
     hipLaunchKernelGGL((head_norm_store_kernel<T, P>), dim3((unsigned)((items + HNS_WAVES - 1) / HNS_WAVES)),
                        dim3(64 * HNS_WAVES), 0, stream, (T*)q_out, q_stride, (const P*)proj, splits, (size_t)split_stride,
