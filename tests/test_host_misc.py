@@ -663,3 +663,20 @@ def test_replay_and_bench_are_commands_of_the_one_command_line(capsys):
     facts = brief()
     assert set(facts) == {"gpu", "arch", "torch", "hip", "rocm", "git", "source"}
     assert len(facts["source"]) == 12 and facts["source"] == source_digest()[:12] == git_info()["source_digest"][:12]
+
+
+def test_the_tile_list_pairs_long_walks_with_short_ones():
+    """Prompt tiles come longest first; where all workgroups are on the device at once, two a unit, the second ones come
+    shortest first, so that the unit with the longest walk also has the shortest."""
+    from turboserve_amd.kernels.ops import Ops
+
+    lens, contexts = [400, 100], [400, 900]
+    plain = Ops.attention_tile_list(lens, contexts)
+    keys = [min(64, lens[r] - (f if r == 0 else f - 400)) + (contexts[r] - lens[r]) + (f if r == 0 else f - 400) for r, f in plain]
+    assert keys == sorted(keys, reverse=True) and len(plain) == 9
+    paired = Ops.attention_tile_list(lens, contexts, heads=4, units=20)
+    assert paired == plain[:5] + plain[:4:-1]
+    # A grid that fits the units once, or that does not fit them twice, keeps its order.
+    assert Ops.attention_tile_list(lens, contexts, heads=4, units=36) == plain
+    assert Ops.attention_tile_list(lens, contexts, heads=4, units=16) == plain
+    assert Ops.attention_tile_list(lens, contexts, heads=64, units=16) == plain

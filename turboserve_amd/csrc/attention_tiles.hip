@@ -16,13 +16,22 @@
 // the transposed value pages as they are, or turned while being staged when they lie in the key
 // rows); the next tile's loads are in flight while this one is computed.  Per wavefront: S (16 rows
 // x 64 keys) = Q K^T by v_mfma_f32_16x16x32_bf16, online softmax in the accumulator layout, P
-// through LDS into the operand layout, O += P V.
+// through LDS into the operand layout, O += P V.  The softmax runs to the base 2 (the scale, slopes, biases and sinks come in
+// multiplied by log2 e); tiles that every row of a wavefront sees whole are not masked, and the sums are rescaled only where
+// a maximum has grown.
 //
 // Sizes: Dk (up to 384; 448 with the values inside the key rows) and Dv (up to 256; 384) multiples of 8; pages of 8 tokens or more (a multiple of 8).
 #include "common.hpp"
 
 typedef __bf16 fa_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float fa_f32x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 fa_bf16x2 __attribute__((ext_vector_type(2)));
+typedef float fa_f32x2 __attribute__((ext_vector_type(2)));
+
+#define FA_LOG2E 1.44269504088896340736f
+#define FA_LN2 0.69314718055994530942f
+
+__device__ __forceinline__ float fa_exp2(float v) { return __builtin_amdgcn_exp2f(v); }
 
 #define FA_ROWS 64
 #define FA_KEYS 64
@@ -160,11 +169,16 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
     const bool live = r < tile_rows;
     pos[i] = live ? row_position(r) : -1;  // an idle row sees nothing
     low[i] = live ? fa_lowest(pos[i], rule.window, rule.chunk) : 0;
-    slope[i] = (slopes && live) ? slopes[row_head(r)] : 0.f;
+    slope[i] = (slopes && live) ? slopes[row_head(r)] * FA_LOG2E : 0.f;
     // The row's line of the bias table (read by distance); an idle row reads head 0's and is masked.
     bias_row[i] = distance_bias ? distance_bias + (size_t)(live ? row_head(r) : 0) * bias_len : nullptr;
-    sink_at[i] = (sink_scores && live) ? sink_scores[row_head(r)] : 0.f;
+    sink_at[i] = (sink_scores && live) ? sink_scores[row_head(r)] * FA_LOG2E : 0.f;
   }
+  // Keys that every live row of the wavefront sees (positions grow with the rows): seen_from .. seen_to.
+  const int wave_last = min(wave * 16 + 15, tile_rows - 1);
+  const int seen_to = row_position(wave * 16), seen_from = fa_lowest(row_position(wave_last), rule.window, rule.chunk);
+  const bool wave_live = wave * 16 < tile_rows;
+  const float scale2 = rule.scale * FA_LOG2E;
   // (Key rows that hold their values have no variant with a bias: the launch refuses it.)
   const bool biased = !VALUES_IN_KEYS && distance_bias != nullptr;
   fa_f32x4 o[VD];
@@ -203,26 +217,35 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
   ts_u32x4 k_reg[K_MINE];
   ts_u32x4 v_reg[VALUES_IN_KEYS ? 1 : V_MINE];
   const int last_key = context - 1;
+  // The key of a piece.  Outside key_lo .. last: a live key again (its page may have been given back, or never taken); masked later.
+  auto key_of = [&](int tile, int j) __attribute__((always_inline)) {
+    const int key = min(tile * FA_KEYS + max(k_key[j], 0), last_key);
+    return key >= keep_end ? max(key, key_lo) : key;
+  };
+  // The first of the eight keys (of one page) of a piece of values: the same for all of a thread's pieces.
+  auto value_key_of = [&](int tile) __attribute__((always_inline)) {
+    const int key = min(tile * FA_KEYS + 8 * (tid % (FA_KEYS / 8)), last_key & ~7);
+    return key >= keep_end ? max(key, key_lo & ~7) : key;
+  };
+  // The pages of a tile's pieces, asked for a tile ahead of the pieces themselves.
+  int k_page[K_MINE], v_page = 0;
+  auto look_up = [&](int tile) __attribute__((always_inline)) {
+#pragma unroll
+    for (int j = 0; j < K_MINE; ++j) k_page[j] = table[key_of(tile, j) >> block_shift];
+    if (!VALUES_IN_KEYS) v_page = table[value_key_of(tile) >> block_shift];
+  };
   auto fetch = [&](int tile) __attribute__((always_inline)) {
-    const int key0 = tile * FA_KEYS;
 #pragma unroll
     for (int j = 0; j < K_MINE; ++j) {
-      // Outside key_lo .. last: a live key again (its page may have been given back, or never taken); masked later.
-      int key = min(key0 + max(k_key[j], 0), last_key);
-      if (key >= keep_end) key = max(key, key_lo);
-      const int page = table[key >> block_shift];
-      const uint16_t* src = k_pages + ((((size_t)page * kv_heads + kvh) << block_shift) + (key & block_mask)) * dk + k_at[j];
+      const uint16_t* src = k_pages + ((((size_t)k_page[j] * kv_heads + kvh) << block_shift) + (key_of(tile, j) & block_mask)) * dk + k_at[j];
       k_reg[j] = k_key[j] >= 0 ? *reinterpret_cast<const ts_u32x4*>(src) : ts_u32x4{0u, 0u, 0u, 0u};
     }
     if (!VALUES_IN_KEYS) {
+      const uint16_t* column = v_pages + ((((size_t)v_page * kv_heads + kvh) * dv) << block_shift) + (value_key_of(tile) & block_mask);
 #pragma unroll
       for (int j = 0; j < V_MINE; ++j) {
         const int piece = tid + j * FA_THREADS;
-        const int d = piece / (FA_KEYS / 8);
-        int key = min(key0 + 8 * (piece % (FA_KEYS / 8)), last_key & ~7);  // eight keys of one page
-        if (key >= keep_end) key = max(key, key_lo & ~7);
-        const int page = table[key >> block_shift];
-        const uint16_t* src = v_pages + ((((size_t)page * kv_heads + kvh) * dv + d) << block_shift) + (key & block_mask);
+        const uint16_t* src = column + ((size_t)(piece / (FA_KEYS / 8)) << block_shift);
         v_reg[j] = piece < v_pieces ? *reinterpret_cast<const ts_u32x4*>(src) : ts_u32x4{0u, 0u, 0u, 0u};
       }
     }
@@ -259,12 +282,19 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
   __syncthreads();
 
   uint16_t* my_p = ps + wave * 16 * P_ROW;
-  if (tile_begin < tile_end) fetch(tile_of(tile_begin));
+  if (tile_begin < tile_end) {
+    look_up(tile_of(tile_begin));
+    fetch(tile_of(tile_begin));
+    look_up(tile_of(min(tile_begin + 1, tile_end - 1)));
+  }
   for (int walk = tile_begin; walk < tile_end; ++walk) {
     __syncthreads();  // everyone has read the tile before
     stage();
     __syncthreads();
-    if (walk + 1 < tile_end) fetch(tile_of(walk + 1));  // in flight while this tile is computed
+    if (walk + 1 < tile_end) {  // in flight while this tile is computed
+      fetch(tile_of(walk + 1));
+      look_up(tile_of(min(walk + 2, tile_end - 1)));
+    }
     const int key0 = tile_of(walk) * FA_KEYS;
     // The biases of this lane's 16 scores, asked for in one stretch ahead of the first product, so
     // that they arrive while it runs (asked for where they are added, each is waited for on its own).
@@ -301,52 +331,77 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
 #pragma unroll
         for (int i = 0; i < 4; ++i) s[ct][i] = rule.softcap / rule.scale * tanhf(s[ct][i] * rule.scale / rule.softcap);
     }
-    // Scores of this lane: row 4 group + i, key key0 + 16 ct + r16.
+    // Scores of this lane: row 4 group + i, key key0 + 16 ct + r16.  (A wavefront without a live row masks nothing: what it
+    // sums up is not written.)
+    const bool whole = !wave_live || (key0 >= seen_from && key0 + FA_KEYS - 1 <= seen_to);
     float tile_max[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) tile_max[i] = -INFINITY;
 #pragma unroll
-    for (int ct = 0; ct < 4; ++ct) {
-      const int key = key0 + 16 * ct + r16;
+    for (int ct = 0; ct < 4; ++ct)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        float v = fmaf(slope[i], (float)(key - pos[i]), s[ct][i] * rule.scale);
-        const bool seen = (key >= low[i] || key < rule.keep) && key <= pos[i];
-        if (biased) v += bias_of[ct][i];
-        v = seen ? v : -INFINITY;
-        s[ct][i] = v;
-        tile_max[i] = fmaxf(tile_max[i], v);
+      for (int i = 0; i < 4; ++i) s[ct][i] *= scale2;
+    if (slopes) {
+#pragma unroll
+      for (int ct = 0; ct < 4; ++ct)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) s[ct][i] = fmaf(slope[i], (float)(key0 + 16 * ct + r16 - pos[i]), s[ct][i]);
+    }
+    if (biased) {
+#pragma unroll
+      for (int ct = 0; ct < 4; ++ct)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) s[ct][i] = fmaf(bias_of[ct][i], FA_LOG2E, s[ct][i]);
+    }
+    if (!whole) {
+#pragma unroll
+      for (int ct = 0; ct < 4; ++ct) {
+        const int key = key0 + 16 * ct + r16;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const bool seen = (key >= low[i] || key < rule.keep) && key <= pos[i];
+          s[ct][i] = seen ? s[ct][i] : -INFINITY;
+        }
       }
     }
-    float alpha[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float v = row16_max(tile_max[i]);
-      const float m_new = fmaxf(m_run[i], v);
-      // A row that has seen nothing yet keeps a zero sum: exp(-inf - -inf) must not be formed.
-      alpha[i] = m_new == -INFINITY ? 1.f : expf(m_run[i] - m_new);
-      m_run[i] = m_new;
+    for (int i = 0; i < 4; ++i) tile_max[i] = row16_max(fmaxf(fmaxf(s[0][i], s[1][i]), fmaxf(s[2][i], s[3][i])));
+    bool grew = false;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) grew = grew || tile_max[i] > m_run[i];
+    if (__any(grew)) {
+      float alpha[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float m_new = fmaxf(m_run[i], tile_max[i]);
+        // A row that has seen nothing yet keeps a zero sum: the exponential of -inf - -inf must not be formed.
+        alpha[i] = m_new == -INFINITY ? 1.f : fa_exp2(m_run[i] - m_new);
+        m_run[i] = m_new;
+        l_run[i] *= alpha[i];
+      }
+#pragma unroll
+      for (int vt = 0; vt < VD; ++vt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[vt][i] *= alpha[i];
     }
     float sum[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int ct = 0; ct < 4; ++ct) {
+    for (int ct = 0; ct < 4; ct += 2) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float p = s[ct][i] == -INFINITY ? 0.f : expf(s[ct][i] - m_run[i]);
-        // The probability as the second product sees it: rounded; the denominator counts the same value.
-        const bf16_t rounded = from_float<bf16_t>(p);
-        sum[i] += to_float(rounded);
-        my_p[(4 * group + i) * P_ROW + 16 * ct + r16] = rounded.bits;
+        // (A row that has seen nothing has no maximum either: its masked scores stand against 0.)
+        const float top = m_run[i] == -INFINITY ? 0.f : m_run[i];
+        const fa_f32x2 p = {fa_exp2(s[ct][i] - top), fa_exp2(s[ct + 1][i] - top)};
+        // The probabilities as the second product sees them: rounded; the denominator counts the same values.
+        const uint32_t rounded = __builtin_bit_cast(uint32_t, __builtin_convertvector(p, fa_bf16x2));
+        sum[i] += __uint_as_float(rounded << 16) + __uint_as_float(rounded & 0xffff0000u);
+        uint16_t* to = my_p + (4 * group + i) * P_ROW + 16 * ct + r16;
+        to[0] = (uint16_t)(rounded & 0xffffu);
+        to[16] = (uint16_t)(rounded >> 16);
       }
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      l_run[i] = l_run[i] * alpha[i] + row16_sum(sum[i]);
-    }
-#pragma unroll
-    for (int vt = 0; vt < VD; ++vt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) o[vt][i] *= alpha[i];
+    for (int i = 0; i < 4; ++i) l_run[i] += row16_sum(sum[i]);
     __builtin_amdgcn_s_waitcnt(0xc07f);  // the wavefront's own LDS writes of P have landed (lgkmcnt 0)
     __builtin_amdgcn_wave_barrier();
     // O += P V over the tile's 64 keys.
@@ -381,7 +436,7 @@ attention_tiles_kernel(uint16_t* __restrict__ out, float* __restrict__ partial_o
       for (int vt = 0; vt < VD; ++vt)
         if (16 * vt + r16 < dv) dst[16 * vt + r16] = o[vt][i];
       if (r16 == 0) {
-        partial_ml[2 * slot] = m_run[i];
+        partial_ml[2 * slot] = m_run[i] * FA_LN2;
         partial_ml[2 * slot + 1] = l_run[i];
       }
     }

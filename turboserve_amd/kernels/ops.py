@@ -1622,11 +1622,13 @@ class Ops:
 
     @staticmethod
     def attention_tile_list(query_lens, context_lens=None, rows: int = 64, *, window: int | None = None,
-                            chunk: int | None = None) -> list[list[int]]:
+                            chunk: int | None = None, heads: int = 0, units: int = 0) -> list[list[int]]:
         """``[request, first row]`` of every tile of ``rows`` consecutive tokens of the requests
         ``0 .. len(query_lens) - 1`` at the front of a step; with the requests' ``context_lens``, the
         tiles that see the most keys (under the layer's ``window`` and ``chunk``) come first, so that
-        the longest walks start first."""
+        the longest walks start first.  Given the layer's ``heads`` (workgroups a tile) and the device's compute ``units``:
+        where all workgroups are on the device at once, two a unit, the second ones come in the opposite order, so that a long
+        walk shares its unit with a short one."""
         tiles, row = [], 0
         for request, count in enumerate(query_lens):
             start = 0 if context_lens is None else context_lens[request] - count
@@ -1637,6 +1639,9 @@ class Ops:
             row += count
         if context_lens is not None:
             tiles.sort(key=lambda tile: -tile[0])
+            once = units // heads if heads else 0
+            if 0 < once < len(tiles) <= 2 * once:
+                tiles[once:] = tiles[:once - 1:-1]
         return [[request, first] for _, request, first in tiles]
 
     def attention_tiles(self, q: torch.Tensor, q_stride: int, k_pages: torch.Tensor, v_pages: torch.Tensor | None,
