@@ -106,7 +106,7 @@ def ints(values):
 LENGTHS, SLOTS = [300, 129, 31], [3, 1, 4]
 
 
-def walked(ops, dtype, width: int, rows: list[torch.Tensor], step, pieces: bool) -> None:
+def walked(ops, rows: list[torch.Tensor], step, pieces: bool) -> None:
     """Feeds three requests side by side, through slots not in row order, in portions of changing size: long ones (cut into
     pieces that are full, one token over, one short), short ones, single tokens behind them.  ``step(given, live, starts, plan)``
     runs one; ``given`` are the rows as partial sums or as the run's type, in turn.  In bfloat16 runs the rows are bfloat16
@@ -180,7 +180,7 @@ def test_a_state_with_a_fixed_decay(ops, dtype, heads, n, p):
     decay = [(0.999, 0.9, 1.0, 0.01, 0.99, 0.7, 0.9999, 0.5)[a] for a in range(heads)]
     pieces = ops.decaying_pieces_supported(dtype, n, p)
     assert pieces == (dtype == torch.bfloat16 and (n, p) in CUT)
-    walked(ops, dtype, width, rows, RetentionStep(ops, dtype, heads, n, p, columns, decay, rows), pieces)
+    walked(ops, rows, RetentionStep(ops, dtype, heads, n, p, columns, decay, rows), pieces)
 
 
 class MemoryStep:
@@ -258,7 +258,7 @@ def test_a_memory_with_exponential_gates(ops, dtype, heads, n, p, gates, cap):
         row[:, width - 2 * heads:width] *= 2.0
     rows = [row.to(dtype) for row in rows]
     pieces = ops.decaying_pieces_supported(dtype, n, p)
-    walked(ops, dtype, width, rows, MemoryStep(ops, dtype, heads, n, p, cap, gates, rows), pieces)
+    walked(ops, rows, MemoryStep(ops, dtype, heads, n, p, cap, gates, rows), pieces)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
